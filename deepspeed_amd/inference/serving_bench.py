@@ -338,6 +338,7 @@ def _lolulorn_kernel_rows(z, dev):
     """(name, like, seconds, bound seconds) per Lolulorn kernel at this size,
     each followed by the like kernel of the Llama path."""
     from ..ops import serving_kernels as sk
+    from ..ops.linear_recurrence import head_norm_gate
     from ..ops.attention import flash_attn_available, flash_attn_fwd
     from ..ops.norms import rms_norm
     from ..ops.paged_attention import paged_decode_attention
@@ -476,7 +477,7 @@ def _lolulorn_kernel_rows(z, dev):
     gate = torch.randn(T, RH * rv, device=dev).to(bf)
     nw = torch.ones(rv, device=dev)
     row("head_norm_gate (fp32 in, bf16 gate and out)", "rms_norm",
-        lambda: sk.head_norm_gate(o32, nw, gate, 1e-6, bf), T * RH * rv * 8)
+        lambda: head_norm_gate(o32, nw, gate, 1e-6, bf), T * RH * rv * 8)
     # ---- activations
     gu = torch.randn(T, 2 * F, device=dev).to(bf)
     row("glu gelu_tanh", "swiglu", lambda: sk.glu(gu, 1), T * F * 6)
@@ -550,6 +551,7 @@ def _savovik_kernel_rows(z, dev):
     the Lolulorn path ("like" names it; rows with an empty "like" are the
     siblings themselves)."""
     from ..ops import serving_kernels as sk
+    from ..ops.linear_recurrence import head_norm_gate
     from ..ops.rope import rope_tables
     from .state_cache import PagedStateCache
     bf = torch.bfloat16
@@ -690,7 +692,7 @@ def _savovik_kernel_rows(z, dev):
     gate2 = torch.randn(T, RH * rv, device=dev).to(bf)
     nw = torch.ones(rv, device=dev)
     row("head_norm_gate (lolulorn)", "",
-        lambda: sk.head_norm_gate(o2, nw, gate2, 1e-6, bf), T * RH * rv * 8)
+        lambda: head_norm_gate(o2, nw, gate2, 1e-6, bf), T * RH * rv * 8)
     del o32, xx, gate, o2, gate2, pj, pj2
     # ---- the scans
     ch, SN = W, 16
@@ -829,6 +831,7 @@ def _numolorn_kernel_rows(z, dev):
     like kernel of the Lolulorn or Fizesun path at the same shapes ("like"
     names it; rows with an empty "like" are the siblings themselves)."""
     from ..ops import serving_kernels as sk
+    from ..ops.linear_recurrence import head_norm_gate
     from ..ops.rope import rope_tables
     from .state_cache import PagedStateCache
     bf = torch.bfloat16
@@ -1038,10 +1041,10 @@ def _numolorn_kernel_rows(z, dev):
     gate = torch.randn(T, RH * rv, device=dev).to(bf)
     nw = torch.ones(rv, device=dev)
     row("head_norm_gate, sigmoid gate", "head_norm_gate",
-        lambda: sk.head_norm_gate(o32, nw, gate, 1e-6, bf, "sigmoid"),
+        lambda: head_norm_gate(o32, nw, gate, 1e-6, bf, "sigmoid"),
         T * RH * rv * 8)
     row("head_norm_gate (lolulorn: silu gate)", "",
-        lambda: sk.head_norm_gate(o32, nw, gate, 1e-6, bf), T * RH * rv * 8)
+        lambda: head_norm_gate(o32, nw, gate, 1e-6, bf), T * RH * rv * 8)
     del o32, gate
     # ---- router and expert activation
     E = z["experts"] + 2

@@ -13,6 +13,7 @@ from .mixtral import (MixtralConfig, MixtralForCausalLM, mixtral_8x7b,
 from .fizesun import FizesunConfig, FizesunForCausalLM, fizesun_tiny
 from .savovik import SavovikConfig, SavovikForCausalLM, savovik_tiny
 from .numolorn import NumolornConfig, NumolornForCausalLM, numolorn_tiny
+from .redudra import RedudraConfig, RedudraForCausalLM, redudra_tiny
 from .registry import (architectures, build_model, load_pretrained,
                        register_architecture)
 
@@ -28,6 +29,7 @@ __all__ = [
     "FizesunConfig", "FizesunForCausalLM", "fizesun_tiny",
     "SavovikConfig", "SavovikForCausalLM", "savovik_tiny",
     "NumolornConfig", "NumolornForCausalLM", "numolorn_tiny",
+    "RedudraConfig", "RedudraForCausalLM", "redudra_tiny",
     "architectures", "build_model", "load_pretrained",
     "register_architecture",
 ]

@@ -216,16 +216,20 @@ class GatedLinearAttention(nn.Module):
 
 
 class GatedMLP(nn.Module):
-    """down(act(gate h) * (up h)); gate and up rows fused."""
+    """down(act(gate h) * (up h)); gate and up rows fused. ``bias``: all
+    three projections have one."""
 
-    def __init__(self, width, ff, act, dtype):
+    def __init__(self, width, ff, act, dtype, bias=False):
         super().__init__()
         self.act = act
         self.w_gu = _w(2 * ff, width, dtype=dtype)
         self.w_down = _w(width, ff, dtype=dtype)
+        self.b_gu = _w(2 * ff, dtype=dtype) if bias else None
+        self.b_down = _w(width, dtype=dtype) if bias else None
 
     def forward(self, h):
-        return F.linear(glu(F.linear(h, self.w_gu), self.act), self.w_down)
+        return F.linear(glu(F.linear(h, self.w_gu, self.b_gu), self.act),
+                        self.w_down, self.b_down)
 
 
 class PostNorm(nn.Module):

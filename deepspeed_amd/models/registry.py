@@ -93,6 +93,7 @@ def _register_builtin():
     from .lolulorn import build_from_config as build_lolulorn
     from .mixtral import MixtralConfig, MixtralForCausalLM
     from .numolorn import build_from_config as build_numolorn
+    from .redudra import build_from_config as build_redudra
     from .savovik import build_from_config as build_savovik
     hf = {"num_hidden_layers": "num_layers",
           "num_attention_heads": "num_heads",
@@ -112,6 +113,7 @@ def _register_builtin():
     register_architecture("Lolulorn", build_lolulorn, wants_tensors=True)
     register_architecture("Savovik", build_savovik)
     register_architecture("Numolorn", build_numolorn, wants_tensors=True)
+    register_architecture("Redudra", build_redudra)
 
 
 _register_builtin()

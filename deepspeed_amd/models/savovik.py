@@ -107,11 +107,21 @@ def _w(*shape, dtype):
     return nn.Parameter(torch.empty(*shape, dtype=dtype), requires_grad=False)
 
 
-def _rot_tables(rot, max_seq, device):
+def rot_tables(rot, max_seq, device):
     """cos/sin tables [max_seq, dims/2] for a mixer's ``rot`` block: plain
     frequencies ``base^(-2i/dims)``; ``scaling`` with ``original`` is the
-    three-band rule, without it every frequency is divided by ``factor``."""
+    three-band rule (``low``, ``high``) or YaRN (``fast``, ``slow``), without
+    it every frequency is divided by ``factor``."""
     sc = rot.get("scaling") or {}
+    if "fast" in sc:
+        return rope_tables(int(rot["dims"]), max_seq, float(rot["base"]),
+                           device=device, rope_scaling={
+                               "rope_type": "yarn",
+                               "factor": float(sc["factor"]),
+                               "beta_fast": float(sc["fast"]),
+                               "beta_slow": float(sc["slow"]),
+                               "original_max_position_embeddings":
+                                   float(sc["original"])})
     if "original" in sc:
         return rope_tables(int(rot["dims"]), max_seq, float(rot["base"]),
                            device=device, rope_scaling={
@@ -127,7 +137,8 @@ def _rot_tables(rot, max_seq, device):
 class GroupedAttention(nn.Module):
     """Grouped-query attention over paged rows; what differs between its two
     uses is given by flags: projection biases, per-head query/key norms, the
-    rotary pairing, unit-RMS values, the score cap and the kind of mask."""
+    rotary pairing, unit-RMS values, the score cap and the kind of mask (a
+    window may keep a sequence's first tokens)."""
 
     def __init__(self, m: dict, eps, dtype, *, bias, qk_norm, layout, v_unit,
                  mask):
@@ -144,6 +155,7 @@ class GroupedAttention(nn.Module):
         self.scale = float(m["scale"])
         self.softcap = float(m.get("softcap") or 0.0)
         size = int((m.get("mask") or {}).get("size", 0))
+        self.keep_first = int((m.get("mask") or {}).get("keep_first", 0))
         self.window = size if mask == "window" else 0
         self.chunk = size if mask == "chunk" else 0
         self.layout = layout
@@ -166,7 +178,7 @@ class GroupedAttention(nn.Module):
         """proj: this step's q|k|v (a column slice is fine). Returns the
         heads' results side by side, before the output projection."""
         b = cache.batch
-        cos, sin = _rot_tables(self.rot, cache.max_seq, proj.device) \
+        cos, sin = rot_tables(self.rot, cache.max_seq, proj.device) \
             if self.rot_dims else (None, None)
         pool = cache.pools[stream]
         q = attn_prep(proj, b, pool, self.q_norm, self.k_norm, self.eps,
@@ -174,8 +186,8 @@ class GroupedAttention(nn.Module):
                       self.rot_dims, cos, sin, True, self.norm, self.layout,
                       self.v_unit_eps)
         return window_attention(q, pool, b, self.kv_heads, self.dim,
-                                self.vdim, self.scale, self.window, 0, None,
-                                self.chunk, self.softcap, out_scale, out)
+                                self.vdim, self.scale, self.window,
+                                self.keep_first, None, self.chunk, self.softcap, out_scale, out)
 
 
 class AttentionMixer(nn.Module):

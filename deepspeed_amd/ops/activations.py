@@ -11,6 +11,7 @@
 * ``act_rows(z, act)``: a plain activation of a projection, ``act`` one of
   "gelu_erf" (``0.5 z (1 + erf(z / sqrt 2))``), "gelu_tanh", "silu"; ``z`` may
   be a column slice of a wider projection.
+* ``softcap_rows(z, cap)``: ``cap * tanh(z / cap)``, returned in fp32.
 All evaluate in fp32 and round once.
 """
 
@@ -80,3 +81,10 @@ def act_rows(z, act):
     else:
         y = F.silu(zf)
     return y.to(z.dtype)
+
+
+def softcap_rows(z, cap):
+    """``cap * tanh(z / cap)`` in fp32 (logits; z any float type)."""
+    if z.is_cuda and _sk().enabled():
+        return _sk().softcap_rows(z, cap)
+    return cap * torch.tanh(z.float() / cap)

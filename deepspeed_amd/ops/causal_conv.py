@@ -62,18 +62,22 @@ def residual_add_stats(x, delta):
     return None
 
 
-def conv_silu_ragged(x, conv_w, state, batch, bias=None, out_dtype=None):
+def conv_silu_ragged(x, conv_w, state, batch, bias=None, out_dtype=None,
+                     act="silu"):
     """Short causal convolution per channel followed by SiLU:
     ``silu(sum_j w[:, j] * x_(t - taps + 1 + j) (+ bias))`` with zeros before
-    a sequence's start (the last column weighs the current token).
+    a sequence's start (the last column weighs the current token);
+    ``act=None`` leaves the activation out.
     x [T, C] (may be a column slice of a wider projection), conv_w [C, taps],
     state [slots, taps-1, C] in x's dtype: a sequence's last ``taps - 1``
     inputs, oldest first, updated in place. Sums and SiLU are fp32; returns
     [T, C] fp32, or rounded once to ``out_dtype``."""
+    if act not in ("silu", None):
+        raise ValueError(f"unknown convolution activation {act!r}")
     out_dtype = out_dtype or torch.float32
     if x.is_cuda and _sk().enabled():
         return _sk().conv_silu_ragged(x, conv_w, state, batch, bias,
-                                      out_dtype)
+                                      out_dtype, act)
     taps = conv_w.shape[1]
     wf = conv_w.float()
     out = torch.empty(x.shape, dtype=out_dtype, device=x.device)
@@ -84,7 +88,9 @@ def conv_silu_ragged(x, conv_w, state, batch, bias=None, out_dtype=None):
         acc = (win * wf).sum(-1)
         if bias is not None:
             acc = acc + bias.float()
-        out[at:at + count] = torch.nn.functional.silu(acc).to(out_dtype)
+        if act == "silu":
+            acc = torch.nn.functional.silu(acc)
+        out[at:at + count] = acc.to(out_dtype)
         if taps > 1:
             state[slot] = hist[-(taps - 1):].to(state.dtype)
         at += count

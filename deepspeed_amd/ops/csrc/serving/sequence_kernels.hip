@@ -979,10 +979,10 @@ __device__ __forceinline__ float4 load4(const bf16* p, int e, int n, bool vec) {
   return x;
 }
 
-template <typename T, int ROWS, bool DELTA, bool CHANNEL_DECAY>
+template <typename T, typename TV, int ROWS, bool DELTA, bool CHANNEL_DECAY>
 __global__ __launch_bounds__(NT) void linear_scan_k(
     const T* __restrict__ q, int ld_q, const T* __restrict__ k, int ld_k,
-    const T* __restrict__ v, int ld_v, const float* __restrict__ decay,
+    const TV* __restrict__ v, int ld_v, const float* __restrict__ decay, int ld_decay,
     const float* __restrict__ beta, float* __restrict__ state, const int* __restrict__ cu,
     const int* __restrict__ seq_slot, float* __restrict__ out, int G, int H, int dim, int vdim,
     float q_scale) {
@@ -1049,7 +1049,7 @@ __global__ __launch_bounds__(NT) void linear_scan_k(
         else if (e == SCAN_COLS)
           x = DELTA ? beta[(int64_t)t * H + h] : 1.f;
         else
-          x = CHANNEL_DECAY ? 1.f : decay[(int64_t)t * H + h];
+          x = CHANNEL_DECAY ? 1.f : decay[(int64_t)t * ld_decay + h];
       }
       ps[i] = x;
     }
@@ -1160,23 +1160,130 @@ __global__ __launch_bounds__(NT) void linear_scan_k(
   }
 }
 
-// out[t, h*vdim + c] = o / sqrt(mean_c(o^2) + eps) * w[c] * act(gate),
-// act = SiLU, or the plain sigmoid with SIGMOID
+// out[t, h*vdim + c] = o / sqrt(mean_c(o^2) + eps) * w[c] * act(gate) *
+// out_scale (w null: no weight), act = SiLU, or the plain sigmoid with SIGMOID
 template <typename T, bool SIGMOID>
 __global__ __launch_bounds__(NT) void head_norm_gate_k(
     const float* __restrict__ o, const float* __restrict__ w, const T* __restrict__ gate,
-    int ld_gate, T* __restrict__ out, int H, int vdim, float eps) {
+    int ld_gate, T* __restrict__ out, int ld_out, int H, int vdim, float eps, float out_scale) {
   const int t = blockIdx.x;
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
   for (int h = wid; h < H; h += NT / 64) {
     const float* oh = o + ((int64_t)t * H + h) * vdim;
     float ss = 0.f;
     for (int c = lane; c < vdim; c += 64) ss += oh[c] * oh[c];
-    const float inv = rsqrtf(wave_sum(ss) / (float)vdim + eps);
+    const float inv = rsqrtf(wave_sum(ss) / (float)vdim + eps) * out_scale;
     for (int c = lane; c < vdim; c += 64) {
       const float gv = ld(gate + (int64_t)t * ld_gate + h * vdim + c);
-      st(out + ((int64_t)t * H + h) * vdim + c,
-         oh[c] * inv * w[c] * (SIGMOID ? sigmoidf_(gv) : siluf_(gv)));
+      st(out + (int64_t)t * ld_out + h * vdim + c,
+         oh[c] * inv * (w ? w[c] : 1.f) * (SIGMOID ? sigmoidf_(gv) : siluf_(gv)));
+    }
+  }
+}
+
+// The same with eight neighbouring columns per lane: LG lanes (a power of two,
+// vdim <= 8 * LG) share a head, so a wave covers 64 / LG heads at a time.
+template <typename T, bool SIGMOID, int LG>
+__global__ __launch_bounds__(NT) void head_norm_gate_vec_k(
+    const float* __restrict__ o, const float* __restrict__ w, const T* __restrict__ gate,
+    int ld_gate, T* __restrict__ out, int ld_out, int64_t heads, int H, int vdim, float eps,
+    float out_scale) {
+  const int l = threadIdx.x % LG;
+  const int c = l * 8;
+  // every lane of a wave walks the same number of rounds: the sums are shuffles
+  for (int64_t j0 = (int64_t)blockIdx.x * (NT / LG); j0 < heads;
+       j0 += (int64_t)gridDim.x * (NT / LG)) {
+    const int64_t j = j0 + threadIdx.x / LG;
+    const bool act = j < heads && c < vdim;
+    float x[8];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) x[e] = 0.f;
+    if (act) load8(o + j * vdim + c, x);
+    float ss = 0.f;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) ss += x[e] * x[e];
+#pragma unroll
+    for (int d = 1; d < LG; d <<= 1) ss += __shfl_xor(ss, d, 64);
+    if (!act) continue;
+    const float inv = rsqrtf(ss / (float)vdim + eps) * out_scale;
+    const int64_t t = j / H;
+    const int at = (int)(j - t * H) * vdim + c;
+    float g[8];
+    load8(gate + t * ld_gate + at, g);
+    if (w) {
+      float wv[8];
+      load8(w + c, wv);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) x[e] *= wv[e];
+    }
+#pragma unroll
+    for (int e = 0; e < 8; ++e) x[e] *= inv * (SIGMOID ? sigmoidf_(g[e]) : siluf_(g[e]));
+    store8(out + t * ld_out + at, x);
+  }
+}
+
+// ---------------------------------------------------- retention prologue
+// qk row (stride ld_qk) = [ q (H x dim) | k (H x dim) ]: rotation of the first
+// rot_dims coordinates of every head (HALF pairs i with i + rot_dims/2, else
+// 2i with 2i+1), keys then times k_scale; float out. VEC: eight neighbouring
+// coordinates per thread.
+template <typename T, bool HALF, bool VEC>
+__global__ __launch_bounds__(NT) void retention_prep_k(
+    const T* __restrict__ qk, int ld_qk, const int* __restrict__ tok_pos,
+    const float* __restrict__ cosT, const float* __restrict__ sinT, float* __restrict__ q_out,
+    float* __restrict__ k_out, int H, int dim, int rot_dims, float k_scale) {
+  const int t = blockIdx.x;
+  const int n = H * dim, half = rot_dims >> 1;
+  const T* p = qk + (int64_t)t * ld_qk;
+  const float* cs = cosT + (int64_t)tok_pos[t] * half;
+  const float* sn = sinT + (int64_t)tok_pos[t] * half;
+  constexpr int E = VEC ? 8 : 1;
+  for (int e0 = threadIdx.x * E; e0 < 2 * n; e0 += NT * E) {
+    const bool is_k = e0 >= n;
+    const int at = is_k ? e0 - n : e0;
+    const int c = at % dim;
+    const T* hd = p + e0 - c;  // the head's first coordinate
+    float* out = (is_k ? k_out : q_out) + (int64_t)t * n + at;
+    const float sc = is_k ? k_scale : 1.f;
+    if (VEC) {
+      float x[8];
+      load8(hd + c, x);
+      if (c < rot_dims) {
+        if (HALF) {  // the partner group sits half the rotated width away
+          const bool second = c >= half;
+          const int f = second ? c - half : c;
+          float o[8], co[8], si[8];
+          load8(hd + (second ? c - half : c + half), o);
+          load8(cs + f, co);
+          load8(sn + f, si);
+#pragma unroll
+          for (int e = 0; e < 8; ++e)
+            x[e] = second ? x[e] * co[e] + o[e] * si[e] : x[e] * co[e] - o[e] * si[e];
+        } else {
+#pragma unroll
+          for (int e = 0; e < 8; e += 2) {
+            if (c + e < rot_dims) {
+              const float co = cs[(c + e) >> 1], si = sn[(c + e) >> 1];
+              const float u = x[e], v = x[e + 1];
+              x[e] = u * co - v * si;
+              x[e + 1] = v * co + u * si;
+            }
+          }
+        }
+      }
+#pragma unroll
+      for (int e = 0; e < 8; ++e) x[e] *= sc;
+      store8(out, x);
+    } else {
+      float v = ld(hd + c);
+      if (c < rot_dims) {
+        const int j = HALF ? (c < half ? c + half : c - half) : (c ^ 1);
+        const int f = HALF ? (c < half ? c : c - half) : (c >> 1);
+        const bool second = HALF ? c >= half : (c & 1);
+        const float o = ld(hd + j), co = cs[f], si = sn[f];
+        v = second ? v * co + o * si : v * co - o * si;
+      }
+      *out = v * sc;
     }
   }
 }
@@ -1248,7 +1355,7 @@ __global__ __launch_bounds__(NT) void attn_prep_heads_k(
   }
 }
 
-// ------------------------------------ short convolution + bias + SiLU, rows
+// ------------------------------ short convolution + bias (+ SiLU), rows
 // x is a column slice (row stride ld_x) of C channels; earlier inputs come
 // from this step's rows, from the slot's tail, or are zero before position 0.
 template <typename T, typename TO>
@@ -1256,7 +1363,7 @@ __global__ __launch_bounds__(NT) void conv_silu_k(
     const T* __restrict__ x, int ld_x, const T* __restrict__ w, const float* __restrict__ bias,
     const T* __restrict__ state, int64_t state_slot_stride, const int* __restrict__ cu,
     const int* __restrict__ seq_slot, const int* __restrict__ tok_seq,
-    const int* __restrict__ tok_pos, TO* __restrict__ out, int C, int taps) {
+    const int* __restrict__ tok_pos, TO* __restrict__ out, int C, int taps, int silu) {
   const int t = blockIdx.x;
   const int s = tok_seq[t];
   const int j = t - cu[s];
@@ -1273,7 +1380,7 @@ __global__ __launch_bounds__(NT) void conv_silu_k(
       acc += ld(w + (int64_t)c * taps + tail - k) * hk;
     }
     if (bias) acc += bias[c];
-    st(out + (int64_t)t * C + c, siluf_(acc));
+    st(out + (int64_t)t * C + c, silu ? siluf_(acc) : acc);
   }
 }
 
@@ -1406,7 +1513,7 @@ __device__ __forceinline__ void conv8_silu(const T* __restrict__ p, int ld,
                                            const T* __restrict__ w,
                                            const float* __restrict__ bias,
                                            const T* __restrict__ sl, int C, int c, int j,
-                                           int pos, float (&acc)[8]) {
+                                           int pos, float (&acc)[8], bool silu = true) {
   constexpr int TAIL = TAPS - 1;
   float wv[8 * TAPS];  // channel-major: wv[e * TAPS + tap]
 #pragma unroll
@@ -1437,8 +1544,10 @@ __device__ __forceinline__ void conv8_silu(const T* __restrict__ p, int ld,
 #pragma unroll
     for (int e = 0; e < 8; ++e) acc[e] += bv[e];
   }
+  if (silu) {
 #pragma unroll
-  for (int e = 0; e < 8; ++e) acc[e] = siluf_(acc[e]);
+    for (int e = 0; e < 8; ++e) acc[e] = siluf_(acc[e]);
+  }
 }
 
 template <typename T, typename TO, int TAPS>
@@ -1446,7 +1555,7 @@ __global__ __launch_bounds__(NT) void conv_silu_vec_k(
     const T* __restrict__ x, int ld_x, const T* __restrict__ w, const float* __restrict__ bias,
     const T* __restrict__ state, int64_t state_slot_stride, const int* __restrict__ cu,
     const int* __restrict__ seq_slot, const int* __restrict__ tok_seq,
-    const int* __restrict__ tok_pos, TO* __restrict__ out, int C) {
+    const int* __restrict__ tok_pos, TO* __restrict__ out, int C, int silu) {
   const int t = blockIdx.x;
   const int s = tok_seq[t];
   const int j = t - cu[s];
@@ -1455,7 +1564,7 @@ __global__ __launch_bounds__(NT) void conv_silu_vec_k(
   const T* p = x + (int64_t)t * ld_x;
   for (int c = (blockIdx.y * NT + threadIdx.x) * 8; c < C; c += gridDim.y * NT * 8) {
     float acc[8];
-    conv8_silu<T, TAPS>(p, ld_x, w, bias, sl, C, c, j, pos, acc);
+    conv8_silu<T, TAPS>(p, ld_x, w, bias, sl, C, c, j, pos, acc, silu != 0);
     store8(out + (int64_t)t * C + c, acc);
   }
 }
@@ -1863,19 +1972,35 @@ int dsv_sigmoid_pow(const void* z, const float* bias, float* out, int dt, int64_
 // largest head size of keys the scan covers
 int dsv_linear_scan_max_dim() { return SCAN_R * 16; }
 
-// q/k/v: dtype dt with row strides in elements; decay [T, H] (channel_decay 0)
-// or [T, H, dim]; beta [T, H] or null (plain form).
+// q/k: dtype dt, v: dtype v_dt, row strides in elements; decay [T, H]
+// (channel_decay 0), one fixed [H] for all tokens (channel_decay 2) or
+// [T, H, dim] (1); beta [T, H] or null (plain form). v of another type than q
+// comes with the plain form and one decay per head only.
 int dsv_linear_scan(const void* q, int ld_q, const void* k, int ld_k, const void* v, int ld_v,
                     const float* decay, int channel_decay, const float* beta, float* state,
                     const int* cu, const int* seq_slot, float* out, int dt, int nseq, int G, int H,
-                    int dim, int vdim, float q_scale, hipStream_t s) {
+                    int dim, int vdim, float q_scale, int v_dt, hipStream_t s) {
   if (dim > dsv_linear_scan_max_dim() || dim < 1 || H % G) return -1;
+  const int ld_decay = channel_decay == 2 ? 0 : H;
+  if (channel_decay == 2) channel_decay = 0;
+  if (v_dt != dt && (beta || channel_decay || dt != 0)) return -2;
   if (nseq <= 0) return 0;
   dim3 grid(nseq, H, (vdim + SCAN_COLS - 1) / SCAN_COLS);
 #define SCAN(ROWS, DELTA, CD)                                                                   \
-  BY_DTYPE(dt, (linear_scan_k<T, ROWS, DELTA, CD><<<grid, NT, 0, s>>>(                           \
-                   (const T*)q, ld_q, (const T*)k, ld_k, (const T*)v, ld_v, decay, beta, state,  \
-                   cu, seq_slot, out, G, H, dim, vdim, q_scale)))
+  BY_DTYPE(dt, (linear_scan_k<T, T, ROWS, DELTA, CD><<<grid, NT, 0, s>>>(                        \
+                   (const T*)q, ld_q, (const T*)k, ld_k, (const T*)v, ld_v, decay, ld_decay,     \
+                   beta, state, cu, seq_slot, out, G, H, dim, vdim, q_scale)))
+#define SCAN_MIXED(ROWS)                                                                        \
+  linear_scan_k<float, bf16, ROWS, false, false><<<grid, NT, 0, s>>>(                            \
+      (const float*)q, ld_q, (const float*)k, ld_k, (const bf16*)v, ld_v, decay, ld_decay, beta, \
+      state, cu, seq_slot, out, G, H, dim, vdim, q_scale)
+  if (v_dt != dt) {
+    if (dim <= SCAN_R * 4) SCAN_MIXED(4);
+    else if (dim <= SCAN_R * 8) SCAN_MIXED(8);
+    else SCAN_MIXED(16);
+    return (int)hipGetLastError();
+  }
+#undef SCAN_MIXED
 #define SCAN_BY_ROWS(DELTA, CD)                   \
   do {                                            \
     if (dim <= SCAN_R * 4) SCAN(4, DELTA, CD);    \
@@ -1891,18 +2016,59 @@ int dsv_linear_scan(const void* q, int ld_q, const void* k, int ld_k, const void
   return (int)hipGetLastError();
 }
 
-// act: 0 = SiLU of the gate, 1 = sigmoid
+// act: 0 = SiLU of the gate, 1 = sigmoid; w null: no weight
 int dsv_head_norm_gate(const float* o, const float* w, const void* gate, int ld_gate, void* out,
-                       int dt, int Ttok, int H, int vdim, float eps, int act, hipStream_t s) {
+                       int ld_out, int dt, int Ttok, int H, int vdim, float eps, float out_scale,
+                       int act, hipStream_t s) {
   if (Ttok <= 0) return 0;
-  if (act == 1)
+  if (act != 0 && act != 1) return -1;
+  const bool vec = vdim % 8 == 0 && vdim <= 512 && ld_gate % 8 == 0 && ld_out % 8 == 0 &&
+                   (uintptr_t)gate % 16 == 0 && (uintptr_t)out % 16 == 0 &&
+                   (uintptr_t)o % 16 == 0;
+#define HNGV(SIG, LG)                                                                           \
+  BY_DTYPE(dt, (head_norm_gate_vec_k<T, SIG, LG>                                                 \
+                <<<nblocks((int64_t)Ttok * H, NT / LG), NT, 0, s>>>(                             \
+                    o, w, (const T*)gate, ld_gate, (T*)out, ld_out, (int64_t)Ttok * H, H, vdim,  \
+                    eps, out_scale)))
+#define HNGV_BY_LG(SIG)               \
+  do {                                \
+    if (vdim <= 64) HNGV(SIG, 8);     \
+    else if (vdim <= 128) HNGV(SIG, 16); \
+    else if (vdim <= 256) HNGV(SIG, 32); \
+    else HNGV(SIG, 64);               \
+  } while (0)
+  if (vec && act == 1) HNGV_BY_LG(true);
+  else if (vec) HNGV_BY_LG(false);
+  else if (act == 1)
     BY_DTYPE(dt, (head_norm_gate_k<T, true><<<Ttok, NT, 0, s>>>(o, w, (const T*)gate, ld_gate,
-                                                                (T*)out, H, vdim, eps)));
-  else if (act == 0)
-    BY_DTYPE(dt, (head_norm_gate_k<T, false><<<Ttok, NT, 0, s>>>(o, w, (const T*)gate, ld_gate,
-                                                                 (T*)out, H, vdim, eps)));
+                                                                (T*)out, ld_out, H, vdim, eps,
+                                                                out_scale)));
   else
-    return -1;
+    BY_DTYPE(dt, (head_norm_gate_k<T, false><<<Ttok, NT, 0, s>>>(o, w, (const T*)gate, ld_gate,
+                                                                 (T*)out, ld_out, H, vdim, eps,
+                                                                 out_scale)));
+#undef HNGV_BY_LG
+#undef HNGV
+  return (int)hipGetLastError();
+}
+
+int dsv_retention_prep(const void* qk, int ld, const int* tok_pos, const float* cosT,
+                       const float* sinT, float* q_out, float* k_out, int dt, int Ttok, int H,
+                       int dim, int rot_dims, float k_scale, int half, hipStream_t s) {
+  if (rot_dims < 0 || (rot_dims & 1) || rot_dims > dim || ld < 2 * H * dim) return -1;
+  if (rot_dims > 0 && (!cosT || !sinT)) return -2;
+  if (Ttok <= 0) return 0;
+  const bool vec = dim % 8 == 0 && ld % 8 == 0 && (uintptr_t)qk % 16 == 0 &&
+                   (half ? rot_dims % 16 == 0 : true);
+#define RPREP(HALF, VEC)                                                                        \
+  BY_DTYPE(dt, (retention_prep_k<T, HALF, VEC><<<Ttok, NT, 0, s>>>(                              \
+                   (const T*)qk, ld, tok_pos, cosT, sinT, q_out, k_out, H, dim, rot_dims,        \
+                   k_scale)))
+  if (half && vec) RPREP(true, true);
+  else if (half) RPREP(true, false);
+  else if (vec) RPREP(false, true);
+  else RPREP(false, false);
+#undef RPREP
   return (int)hipGetLastError();
 }
 
@@ -1970,7 +2136,8 @@ int dsv_attn_prep_heads(const void* proj, int ld_proj, const float* wq, const fl
 int dsv_conv_silu(const void* x, int ld_x, const void* w, const float* bias, void* state,
                   int64_t state_slot_stride, const int* cu, const int* seq_slot,
                   const int* seq_start, const int* tok_seq, const int* tok_pos, void* out,
-                  int dt, int out_dt, int Ttok, int nseq, int C, int taps, hipStream_t s) {
+                  int dt, int out_dt, int Ttok, int nseq, int C, int taps, int silu,
+                  hipStream_t s) {
   if (taps < 1 || taps > MAXTAPS_SEQ || ld_x < C) return -1;
   if (Ttok <= 0) return 0;
   const bool vec = C % 8 == 0 && ld_x % 8 == 0 && state_slot_stride % 8 == 0 &&
@@ -1981,11 +2148,12 @@ int dsv_conv_silu(const void* x, int ld_x, const void* w, const float* bias, voi
     if (out_dt == 0)                                                                            \
       BY_DTYPE(dt, (conv_silu_vec_k<T, float, TAPS><<<grid, NT, 0, s>>>(                         \
                        (const T*)x, ld_x, (const T*)w, bias, (const T*)state,                   \
-                       state_slot_stride, cu, seq_slot, tok_seq, tok_pos, (float*)out, C)));    \
+                       state_slot_stride, cu, seq_slot, tok_seq, tok_pos, (float*)out, C,       \
+                       silu)));                                                                 \
     else                                                                                        \
       BY_DTYPE(dt, (conv_silu_vec_k<T, T, TAPS><<<grid, NT, 0, s>>>(                             \
                        (const T*)x, ld_x, (const T*)w, bias, (const T*)state,                   \
-                       state_slot_stride, cu, seq_slot, tok_seq, tok_pos, (T*)out, C)));        \
+                       state_slot_stride, cu, seq_slot, tok_seq, tok_pos, (T*)out, C, silu)));  \
   } while (0)
   if (vec && taps == 4) CONVV(4);
   else if (vec && taps == 3) CONVV(3);
@@ -1994,11 +2162,11 @@ int dsv_conv_silu(const void* x, int ld_x, const void* w, const float* bias, voi
 #undef CONVV
     BY_DTYPE(dt, (conv_silu_k<T, float><<<Ttok, NT, 0, s>>>(
                      (const T*)x, ld_x, (const T*)w, bias, (const T*)state, state_slot_stride,
-                     cu, seq_slot, tok_seq, tok_pos, (float*)out, C, taps)));
+                     cu, seq_slot, tok_seq, tok_pos, (float*)out, C, taps, silu)));
   else
     BY_DTYPE(dt, (conv_silu_k<T, T><<<Ttok, NT, 0, s>>>(
                      (const T*)x, ld_x, (const T*)w, bias, (const T*)state, state_slot_stride,
-                     cu, seq_slot, tok_seq, tok_pos, (T*)out, C, taps)));
+                     cu, seq_slot, tok_seq, tok_pos, (T*)out, C, taps, silu)));
   if (taps > 1)
     BY_DTYPE(dt, (conv_tail_shift_k<T><<<nseq, NT, 0, s>>>((const T*)x, ld_x, (T*)state,
                                                            state_slot_stride, cu, seq_slot,

@@ -125,6 +125,298 @@ __global__ __launch_bounds__(NT) void layer_norm_vec_k(
   }
 }
 
+// --------------------------------- residual add + layer norm + token shift
+// v = x[r] + mult * y[r] + extra (y, extra optional), h = layer norm of v with
+// weight and bias; x_out[r] (optional) = v. SHIFT: out[t] = h_t + (h_(t-1) -
+// h_t) * mu, where h_(t-1) is the row before in the same sequence: recomputed
+// from x and y for a block's first row (which is why x_out must not be x when
+// anything is added), from state[slot] for a step's first row of a sequence
+// that holds tokens already, zero at position 0. The block that owns a
+// sequence's first row of the step also stores the sequence's LAST row in
+// state[slot]: it alone reads the old one, and each column is read and written
+// by the same thread. Without SHIFT `idx` (optional) gathers rows.
+//
+// A block takes R consecutive rows, eight columns per thread and group, all
+// rows (and the neighbour row) in registers at once, so their loads and their
+// reductions overlap.
+template <int N>
+__device__ __forceinline__ void block_sum_n(float (&v)[N], float* scratch) {
+  const int nw = blockDim.x >> 6;
+#pragma unroll
+  for (int i = 0; i < N; ++i) v[i] = wave_sum(v[i]);
+  if ((threadIdx.x & 63) == 0) {
+#pragma unroll
+    for (int i = 0; i < N; ++i) scratch[(threadIdx.x >> 6) * N + i] = v[i];
+  }
+  __syncthreads();
+#pragma unroll
+  for (int i = 0; i < N; ++i) {
+    float t = 0.f;
+    for (int k = 0; k < nw; ++k) t += scratch[k * N + i];
+    v[i] = t;
+  }
+  __syncthreads();
+}
+
+template <typename TY, int G>
+__device__ __forceinline__ void resid_row(const float* __restrict__ x, const TY* __restrict__ y,
+                                          float mult, const float* __restrict__ extra,
+                                          int64_t row, int C, float (&v)[G][8]) {
+#pragma unroll
+  for (int i = 0; i < G; ++i) {
+    const int c = (threadIdx.x + i * blockDim.x) * 8;
+    if (c < C) {
+      load8(x + row * C + c, v[i]);
+      if (y) {
+        float t[8];
+        load8(y + row * C + c, t);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[i][e] += mult * t[e];
+      }
+      if (extra) {
+        float t[8];
+        load8(extra + c, t);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[i][e] += t[e];
+      }
+    } else {
+#pragma unroll
+      for (int e = 0; e < 8; ++e) v[i][e] = 0.f;
+    }
+  }
+}
+
+// layer norm of N rows held in registers
+template <int N, int G>
+__device__ __forceinline__ void norm_rows(float (&v)[N][G][8], const float* __restrict__ w,
+                                          const float* __restrict__ b, int C, float eps,
+                                          float* red) {
+  float s[N];
+#pragma unroll
+  for (int j = 0; j < N; ++j) {
+    s[j] = 0.f;
+#pragma unroll
+    for (int i = 0; i < G; ++i)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) s[j] += v[j][i][e];
+  }
+  block_sum_n<N>(s, red);
+  const float rc = 1.f / (float)C;
+  float q[N];
+#pragma unroll
+  for (int j = 0; j < N; ++j) {
+    const float mean = s[j] * rc;
+    q[j] = 0.f;
+#pragma unroll
+    for (int i = 0; i < G; ++i) {
+      if ((threadIdx.x + i * blockDim.x) * 8 < C) {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+          v[j][i][e] -= mean;
+          q[j] += v[j][i][e] * v[j][i][e];
+        }
+      }
+    }
+  }
+  block_sum_n<N>(q, red);
+#pragma unroll
+  for (int j = 0; j < N; ++j) q[j] = rsqrtf(q[j] * rc + eps);
+#pragma unroll
+  for (int i = 0; i < G; ++i) {
+    const int c = (threadIdx.x + i * blockDim.x) * 8;
+    if (c < C) {
+      float wv[8], bv[8];
+      load8(w + c, wv);
+      load8(b + c, bv);
+#pragma unroll
+      for (int j = 0; j < N; ++j)
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[j][i][e] = v[j][i][e] * q[j] * wv[e] + bv[e];
+    }
+  }
+}
+
+template <typename TY, typename TO, bool SHIFT, int G, int R>
+__global__ __launch_bounds__(NT) void residual_norm_vec_k(
+    const float* x, const TY* __restrict__ y, float mult, const float* __restrict__ extra,
+    const float* __restrict__ w, const float* __restrict__ b, float* x_out,
+    const int64_t* __restrict__ idx, const float* __restrict__ mu, float* __restrict__ state,
+    const int* __restrict__ cu, const int* __restrict__ seq_slot,
+    const int* __restrict__ seq_start, const int* __restrict__ tok_seq, TO* __restrict__ out,
+    int rows, int C, float eps) {
+  constexpr int S = SHIFT ? 1 : 0, N = R + S;
+  __shared__ float red[NT / 64 * N];
+  const int row0 = blockIdx.x * R;
+  const int nr = min(R, rows - row0);
+  float v[N][G][8];
+  if (SHIFT) {  // the row before, when it belongs to the same sequence
+    const bool have = row0 > 0 && cu[tok_seq[row0]] != row0;
+    resid_row<TY, G>(x, y, mult, extra, have ? row0 - 1 : row0, C, v[0]);
+  }
+#pragma unroll
+  for (int j = 0; j < R; ++j) {
+    const int r = row0 + min(j, nr - 1);
+    const int64_t src = idx ? idx[r] : r;
+    resid_row<TY, G>(x, y, mult, extra, src, C, v[j + S]);
+    if (x_out && j < nr) {
+#pragma unroll
+      for (int i = 0; i < G; ++i) {
+        const int c = (threadIdx.x + i * blockDim.x) * 8;
+        if (c < C) store8(x_out + (int64_t)r * C + c, v[j + S][i]);
+      }
+    }
+  }
+  norm_rows<N, G>(v, w, b, C, eps, red);
+#pragma unroll
+  for (int j = 0; j < R; ++j) {
+    if (j >= nr) break;
+    const int r = row0 + j;
+    int s = 0;
+    bool first = false, carried = false;
+    if (SHIFT) {
+      s = tok_seq[r];
+      first = cu[s] == r;
+      carried = first && seq_start[s] > 0;
+    }
+#pragma unroll
+    for (int i = 0; i < G; ++i) {
+      const int c = (threadIdx.x + i * blockDim.x) * 8;
+      if (c >= C) continue;
+      float o[8];
+      if (SHIFT) {
+        float p[8], m[8];
+        load8(mu + c, m);
+        if (carried) {
+          load8(state + (int64_t)seq_slot[s] * C + c, p);
+        } else {
+#pragma unroll
+          for (int e = 0; e < 8; ++e) p[e] = first ? 0.f : v[j][i][e];
+        }
+#pragma unroll
+        for (int e = 0; e < 8; ++e) o[e] = v[j + S][i][e] + (p[e] - v[j + S][i][e]) * m[e];
+      } else {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) o[e] = v[j + S][i][e];
+      }
+      store8(out + (int64_t)r * C + c, o);
+    }
+  }
+  if (SHIFT) {
+    // sequences that start in this block: keep their last row of the step
+#pragma unroll
+    for (int j = 0; j < R; ++j) {
+      if (j >= nr) break;
+      const int s = tok_seq[row0 + j];
+      if (cu[s + 1] - 1 != row0 + j || cu[s] < row0) continue;
+#pragma unroll
+      for (int i = 0; i < G; ++i) {
+        const int c = (threadIdx.x + i * blockDim.x) * 8;
+        if (c < C) store8(state + (int64_t)seq_slot[s] * C + c, v[j + S][i]);
+      }
+    }
+    const int s = tok_seq[row0 + nr - 1];
+    const int last = cu[s + 1] - 1;
+    if (cu[s] >= row0 && last >= row0 + nr) {  // it ends in a later block
+      float t[1][G][8];
+      resid_row<TY, G>(x, y, mult, extra, last, C, t[0]);
+      norm_rows<1, G>(t, w, b, C, eps, red);
+#pragma unroll
+      for (int i = 0; i < G; ++i) {
+        const int c = (threadIdx.x + i * blockDim.x) * 8;
+        if (c < C) store8(state + (int64_t)seq_slot[s] * C + c, t[0][i]);
+      }
+    }
+  }
+}
+
+// The same for any C: one row per block, rows read again in every pass.
+template <typename TY, typename TO>
+__global__ __launch_bounds__(NT) void residual_norm_k(
+    const float* x, const TY* __restrict__ y, float mult, const float* __restrict__ extra,
+    const float* __restrict__ w, const float* __restrict__ b, float* x_out,
+    const int64_t* __restrict__ idx, const float* __restrict__ mu, float* __restrict__ state,
+    const int* __restrict__ cu, const int* __restrict__ seq_slot,
+    const int* __restrict__ seq_start, const int* __restrict__ tok_seq, TO* __restrict__ out,
+    int rows, int C, float eps) {
+  __shared__ float red[NT / 64];
+  const int r = blockIdx.x;
+  const int64_t src = idx ? idx[r] : r;
+  auto at = [&](int64_t row, int c) {
+    float t = x[row * C + c];
+    if (y) t += mult * ld(y + row * C + c);
+    if (extra) t += extra[c];
+    return t;
+  };
+  auto stats = [&](int64_t row, float& mean, float& inv) {
+    float a = 0.f;
+    for (int c = threadIdx.x; c < C; c += NT) a += at(row, c);
+    mean = block_sum(a, red) / (float)C;
+    a = 0.f;
+    for (int c = threadIdx.x; c < C; c += NT) {
+      const float d = at(row, c) - mean;
+      a += d * d;
+    }
+    inv = rsqrtf(block_sum(a, red) / (float)C + eps);
+  };
+  float mean, inv, pm = 0.f, pi = 0.f, lm = 0.f, li = 0.f;
+  stats(src, mean, inv);
+  int s = 0, last = 0;
+  bool first = false, carried = false;
+  if (mu) {
+    s = tok_seq[r];
+    first = cu[s] == r;
+    carried = first && seq_start[s] > 0;
+    last = cu[s + 1] - 1;
+    if (!first) stats(r - 1, pm, pi);
+    if (first) {
+      if (last == r) {
+        lm = mean;
+        li = inv;
+      } else {
+        stats(last, lm, li);
+      }
+    }
+  }
+  for (int c = threadIdx.x; c < C; c += NT) {
+    const float nv = at(src, c);
+    const float h = (nv - mean) * inv * w[c] + b[c];
+    float o = h;
+    if (mu) {
+      float* sl = state + (int64_t)seq_slot[s] * C + c;
+      float p = 0.f;
+      if (carried)
+        p = *sl;
+      else if (!first)
+        p = (at(r - 1, c) - pm) * pi * w[c] + b[c];
+      o = h + (p - h) * mu[c];
+      if (first) *sl = last == r ? h : (at(last, c) - lm) * li * w[c] + b[c];
+    }
+    if (x_out) x_out[(int64_t)r * C + c] = nv;
+    st(out + (int64_t)r * C + c, o);
+  }
+}
+
+// cap * tanh(z / cap), float out
+template <typename T, bool VEC>
+__global__ void softcap_rows_k(const T* __restrict__ z, float* __restrict__ out, int64_t n,
+                               float cap) {
+  const float rc = 1.f / cap;
+  if (VEC) {
+    for (int64_t i = (blockIdx.x * (int64_t)blockDim.x + threadIdx.x) * 8; i < n;
+         i += (int64_t)gridDim.x * blockDim.x * 8) {
+      float v[8];
+      load8(z + i, v);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) v[e] = cap * tanhf(v[e] * rc);
+      store8(out + i, v);
+    }
+  } else {
+    for (int64_t i = blockIdx.x * (int64_t)blockDim.x + threadIdx.x; i < n;
+         i += (int64_t)gridDim.x * blockDim.x)
+      out[i] = cap * tanhf(ld(z + i) / cap);
+  }
+}
+
 // out[r] = table[ids[r]] * scale (+ table2[ids2[r]]) (fp32)
 template <typename T>
 __global__ __launch_bounds__(NT) void embed_rows_k(
@@ -1026,6 +1318,67 @@ int dsv_layer_norm(const void* in, int in_dt, const int64_t* idx, const float* w
     else LN(bf16, bf16, false);
   }
 #undef LN
+  return (int)hipGetLastError();
+}
+
+// x_out null: the sum is not stored; mu null: no shift (and x_out may be x)
+int dsv_residual_norm(const float* x, const void* y, int y_dt, float mult, const float* extra,
+                      const float* w, const float* b, float* x_out, const int64_t* idx,
+                      const float* mu, float* state, const int* cu, const int* seq_slot,
+                      const int* seq_start, const int* tok_seq, void* out, int out_dt, int rows,
+                      int C, float eps, hipStream_t s) {
+  if (rows <= 0) return 0;
+  if (C < 1 || !out) return -1;
+  if (mu && (idx || !state || !cu || !seq_slot || !seq_start || !tok_seq)) return -2;
+  if (mu && x_out == x) return -3;
+  if (idx && x_out) return -4;
+  const bool vec = C % 8 == 0 && C <= 8 * NT * 4;
+  int nt = (C / 8 + 63) / 64 * 64;
+  nt = nt < 64 ? 64 : (nt > NT ? NT : nt);
+  const int g = (C / 8 + nt - 1) / nt;
+#define RN_(TY, TO, SH, G, R)                                                                   \
+  residual_norm_vec_k<TY, TO, SH, G, R><<<(rows + R - 1) / R, nt, 0, s>>>(                       \
+      x, (const TY*)y, mult, extra, w, b, x_out, idx, mu, state, cu, seq_slot, seq_start,       \
+      tok_seq, (TO*)out, rows, C, eps)
+#define RN(TY, TO)                                                                              \
+  do {                                                                                          \
+    if (!vec)                                                                                   \
+      residual_norm_k<TY, TO><<<rows, NT, 0, s>>>(x, (const TY*)y, mult, extra, w, b, x_out,     \
+                                                  idx, mu, state, cu, seq_slot, seq_start,      \
+                                                  tok_seq, (TO*)out, rows, C, eps);             \
+    else if (mu && rows >= 2048 && g == 1)                                                      \
+      RN_(TY, TO, true, 1, 4);                                                                  \
+    else if (mu && rows >= 2048 && g == 2)                                                      \
+      RN_(TY, TO, true, 2, 4);                                                                  \
+    else if (mu && g <= 2)                                                                      \
+      RN_(TY, TO, true, 2, 1);                                                                  \
+    else if (mu)                                                                                \
+      RN_(TY, TO, true, 4, 1);                                                                  \
+    else if (g == 1)                                                                            \
+      RN_(TY, TO, false, 1, 1);                                                                 \
+    else if (g == 2)                                                                            \
+      RN_(TY, TO, false, 2, 1);                                                                 \
+    else                                                                                        \
+      RN_(TY, TO, false, 4, 1);                                                                 \
+  } while (0)
+  if (y_dt == 0 && out_dt == 0) RN(float, float);
+  else if (y_dt == 0) RN(float, bf16);
+  else if (out_dt == 0) RN(bf16, float);
+  else RN(bf16, bf16);
+#undef RN
+#undef RN_
+  return (int)hipGetLastError();
+}
+
+int dsv_softcap_rows(const void* z, float* out, int dt, int64_t n, float cap, hipStream_t s) {
+  if (n <= 0) return 0;
+  if (!(cap > 0.f)) return -1;
+  if (n % 8 == 0 && (uintptr_t)z % 16 == 0)
+    BY_DTYPE(dt, (softcap_rows_k<T, true><<<nblocks(n / 8, 256), 256, 0, s>>>((const T*)z, out, n,
+                                                                              cap)));
+  else
+    BY_DTYPE(dt, (softcap_rows_k<T, false><<<nblocks(n, 256), 256, 0, s>>>((const T*)z, out, n,
+                                                                           cap)));
   return (int)hipGetLastError();
 }
 

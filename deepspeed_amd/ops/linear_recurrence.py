@@ -32,13 +32,16 @@ Around the scan:
 * ``softplus_decay``: ``exp(-exp(A_log_h) * softplus(z + bias))`` per head and
   key channel (the delta rule with a decay of its own for every row of S).
 * ``head_norm_gate``: per-head RMS norm of the read-out times a weight shared
-  by the heads, times ``silu(gate)`` or ``sigmoid(gate)``.
+  by the heads (or none), times ``silu(gate)`` or ``sigmoid(gate)``.
+* ``retention_prep``: queries and keys of a retention layer (the plain form
+  with one fixed decay per head): partial rotary positions, keys scaled.
 """
 
 import torch
 import torch.nn.functional as F
 
 from .causal_conv import conv_silu_ragged
+from .rope import rope_half_, rope_interleaved_
 
 UNIT_EPS = 1e-6
 
@@ -112,14 +115,16 @@ def sigmoid_pow(z, bias, inv_tau):
 
 def linear_scan(q, k, v, decay, beta, state, batch, q_scale=1.0):
     """q, k [T, G, dim]; v [T, H, vdim] (head h reads q/k head h // (H/G));
-    decay [T, H] or [T, H, dim] fp32; beta [T, H] fp32 or None;
+    decay fp32: [T, H] or [T, H, dim], or [H] (one fixed number per head);
+    beta [T, H] fp32 or None;
     state [slots, H, dim, vdim] fp32, updated in place. q, k, v may be
-    strided views (last axis contiguous). Returns o [T, H, vdim] fp32."""
+    strided views (last axis contiguous); q and k share a dtype, v may have
+    another. Returns o [T, H, vdim] fp32."""
     T, G, dim = q.shape
     H, vdim = v.shape[1], v.shape[2]
     assert H % G == 0 and state.dtype == torch.float32
     assert state.shape[1:] == (H, dim, vdim)
-    assert decay.shape in ((T, H), (T, H, dim))
+    assert decay.shape in ((H,), (T, H), (T, H, dim))
     if q.is_cuda and _sk().enabled():
         return _sk().linear_scan(q, k, v, decay, beta, state, batch, q_scale)
     rep = H // G
@@ -127,6 +132,8 @@ def linear_scan(q, k, v, decay, beta, state, batch, q_scale=1.0):
     kf = k.float().repeat_interleave(rep, 1)
     vf = v.float()
     dec = decay.float()
+    if dec.dim() == 1:
+        dec = dec.expand(T, H)
     dec = dec[:, :, None, None] if dec.dim() == 2 else dec[:, :, :, None]
     out = torch.empty(T, H, vdim, dtype=torch.float32, device=q.device)
     at = 0
@@ -145,19 +152,28 @@ def linear_scan(q, k, v, decay, beta, state, batch, q_scale=1.0):
     return out
 
 
-def head_norm_gate(o, weight, gate, eps, out_dtype, act="silu"):
-    """o [T, H, vdim] fp32; weight [vdim]; gate [T, H*vdim] pre-activation
-    (may be a column slice). Returns
-    ``o / sqrt(mean_v(o^2) + eps) * weight * act(gate)`` as
-    [T, H*vdim] ``out_dtype``; ``act`` is "silu" or "sigmoid"."""
+def head_norm_gate(o, weight, gate, eps, out_dtype, act="silu",
+                   out_scale=1.0, out=None):
+    """o [T, H, vdim] fp32; weight [vdim] or None (no weight); gate
+    [T, H*vdim] pre-activation (may be a column slice). Returns
+    ``o / sqrt(mean_v(o^2) + eps) * weight * act(gate) * out_scale`` as
+    [T, H*vdim] ``out_dtype``; ``act`` is "silu" or "sigmoid"; ``out`` (a view
+    with contiguous rows) receives the result when given."""
     T, H, vdim = o.shape
+    if out is None:
+        out = torch.empty(T, H * vdim, dtype=out_dtype, device=o.device)
+    assert out.shape == (T, H * vdim) and out.stride(1) == 1 \
+        and out.dtype == out_dtype
     if act not in ("silu", "sigmoid"):
         raise ValueError(f"unknown gate activation {act!r}")
     if o.is_cuda and _sk().enabled():
-        return _sk().head_norm_gate(o, weight, gate, eps, out_dtype, act)
-    y = o * torch.rsqrt(o.pow(2).mean(-1, keepdim=True) + eps) * weight.float()
+        return _sk().head_norm_gate(o, weight, gate, eps, act, out_scale, out)
+    y = o * torch.rsqrt(o.pow(2).mean(-1, keepdim=True) + eps)
+    if weight is not None:
+        y = y * weight.float()
     g = F.silu(gate.float()) if act == "silu" else torch.sigmoid(gate.float())
-    return (y.reshape(T, H * vdim) * g).to(out_dtype)
+    out.copy_(y.reshape(T, H * vdim) * g * out_scale)
+    return out
 
 
 def ssd_prep(proj, batch, conv_w, conv_b, conv_state, a_log, dt_bias, heads,
@@ -203,3 +219,23 @@ def gate_group_norm(o, x, skip, gate, weight, parts, eps, out_dtype):
     y = y.reshape(T, parts, n // parts)
     y = y * torch.rsqrt(y.pow(2).mean(-1, keepdim=True) + eps)
     return (y.reshape(T, n) * weight.float()).to(out_dtype)
+
+
+def retention_prep(proj, batch, heads, dim, rot_dims, cos, sin, k_scale,
+                   layout="half"):
+    """proj [T, 2*heads*dim] = q | k (may be a column slice). Rotates the first
+    ``rot_dims`` coordinates of every head ("half" pairs i with
+    i + rot_dims/2, "interleaved" 2i with 2i+1) and then multiplies the keys
+    by ``k_scale``. Returns fp32 q, k [T, heads, dim]."""
+    T, n = proj.shape[0], heads * dim
+    assert proj.shape[1] == 2 * n and layout in ("half", "interleaved")
+    if proj.is_cuda and _sk().enabled():
+        return _sk().retention_prep(proj, batch, heads, dim, rot_dims, cos,
+                                    sin, k_scale, layout)
+    rotate = rope_interleaved_ if layout == "interleaved" else rope_half_
+    q = proj[:, :n].float().reshape(T, heads, dim).clone()
+    k = proj[:, n:].float().reshape(T, heads, dim).clone()
+    if rot_dims:
+        rotate(q, batch.tok_pos, cos, sin, rot_dims)
+        rotate(k, batch.tok_pos, cos, sin, rot_dims)
+    return q, k * k_scale

@@ -286,3 +286,51 @@ def scaled_add_(x, s1=None, y1=None, s2=None, y2=None, extra=None,
     h1 = (n * norm_w1.float()).to(out_dtype)
     h2 = None if norm_w2 is None else (n * norm_w2.float()).to(out_dtype)
     return h1, h2
+
+
+def residual_norm(x, y, mult, weight, bias, eps, out_dtype=None, extra=None,
+                  shift=None, state=None, batch=None, index=None):
+    """Pre-norm residual step on an fp32 stream: ``x' = x + mult * y (+ extra)``
+    and the layer norm (weight and bias) of the new rows, in one pass.
+
+    ``y`` ([T, C], any float type) may be None (``mult`` is then unused);
+    ``extra`` is one fp32 row [C] added to every token. With ``shift`` ([C],
+    fp32) the normed row h_t becomes ``h_t + (h_(t-1) - h_t) * shift``, where
+    h_(t-1) is the sequence's previous normed row before this mixing: it comes
+    from this step's rows of ``batch``, from ``state[slot]`` ([slots, C] fp32,
+    updated in place to each sequence's last row) or is zero at position 0.
+    With ``index`` (int64 [R], no ``shift``) only those rows are added and
+    normed and the stream is left as it is. All sums are fp32; the normed rows
+    are rounded once to ``out_dtype``.
+
+    Returns (x', h). x' shares x's storage unless ``shift`` is given together
+    with something to add (a row's neighbour must still be read unchanged)."""
+    assert x.dtype == torch.float32
+    assert shift is None or (index is None and batch is not None
+                             and state is not None)
+    out_dtype = out_dtype or torch.float32
+    if x.is_cuda and _sk().enabled():
+        return _sk().residual_norm(x, y, mult, weight, bias, eps, out_dtype,
+                                   extra, shift, state, batch, index)
+    new = x if index is None else x[index]
+    if y is not None:
+        new = new + mult * (y if index is None else y[index]).float()
+    if extra is not None:
+        new = new + extra.float()
+    d = new - new.mean(-1, keepdim=True)
+    h = d * torch.rsqrt((d * d).mean(-1, keepdim=True) + eps) \
+        * weight.float() + bias.float()
+    if shift is not None:
+        prev = torch.zeros_like(h)
+        prev[1:] = h[:-1]
+        at = 0
+        for slot, start, count in zip(batch.slots, batch.starts,
+                                      batch.counts):
+            if count:
+                prev[at] = state[slot] if start > 0 else 0.0
+                state[slot] = h[at + count - 1]
+            at += count
+        h = h + (prev - h) * shift.float()
+    if index is None and new is not x and shift is None:
+        new = x.copy_(new)
+    return (x if index is not None else new), h.to(out_dtype)

@@ -8,6 +8,8 @@ guide: on-device trig turns this memory-bound op VALU-bound) and cached per
 
 from typing import Optional
 
+import math
+
 import torch
 
 from ._loader import get_ext
@@ -34,18 +36,49 @@ def llama3_scale_freqs(inv_freq: torch.Tensor, factor: float = 8.0,
     return torch.where(mid, smoothed, scaled)
 
 
+def yarn_scale_freqs(inv_freq: torch.Tensor, dim: int, theta: float,
+                     factor: float, original_max_position: int,
+                     beta_fast: float = 32.0, beta_slow: float = 1.0):
+    """YaRN (Peng et al., "YaRN: Efficient Context Window Extension of Large
+    Language Models"): pairs that turn more than ``beta_fast`` times within
+    the original context keep their frequency, pairs that turn less than
+    ``beta_slow`` times are divided by ``factor``, with a linear ramp over the
+    pair index between the two. Returns (frequencies, factor on cos and sin).
+    """
+    def turn_dim(turns):
+        return dim * math.log(original_max_position / (2 * math.pi * turns)) \
+            / (2 * math.log(theta))
+
+    lo = max(math.floor(turn_dim(beta_fast)), 0)
+    hi = min(math.ceil(turn_dim(beta_slow)), dim - 1)
+    i = torch.arange(inv_freq.numel(), dtype=inv_freq.dtype)
+    ramp = ((i - lo) / max(hi - lo, 0.001)).clamp(0, 1)
+    return inv_freq / factor * ramp + inv_freq * (1 - ramp), \
+        0.1 * math.log(factor) + 1.0
+
+
 def rope_tables(dim: int, max_seq: int, theta: float = 500000.0,
                 device=None, scaling: float = 1.0, rope_scaling=None):
     """fp32 [max_seq, dim/2] cos/sin tables (Llama-3 default theta).
     ``scaling`` divides positions (linear/PI scaling); ``rope_scaling``
     is a llama3-style dict {factor, low_freq_factor, high_freq_factor,
-    original_max_position_embeddings} applied to the frequencies."""
+    original_max_position_embeddings} applied to the frequencies, or with
+    ``rope_type`` "yarn" {factor, beta_fast, beta_slow,
+    original_max_position_embeddings}, whose tables also carry YaRN's factor
+    on cos and sin."""
     rs_key = tuple(sorted(rope_scaling.items())) if rope_scaling else None
     key = (dim, max_seq, theta, str(device), scaling, rs_key)
     if key not in _table_cache:
         inv_freq = 1.0 / (theta ** (torch.arange(0, dim, 2,
                                                  dtype=torch.float64) / dim))
-        if rope_scaling:
+        mag = 1.0
+        if rope_scaling and rope_scaling.get("rope_type") == "yarn":
+            inv_freq, mag = yarn_scale_freqs(
+                inv_freq, dim, theta, float(rope_scaling["factor"]),
+                rope_scaling["original_max_position_embeddings"],
+                float(rope_scaling.get("beta_fast", 32.0)),
+                float(rope_scaling.get("beta_slow", 1.0)))
+        elif rope_scaling:
             inv_freq = llama3_scale_freqs(
                 inv_freq,
                 factor=float(rope_scaling.get("factor", 8.0)),
@@ -57,8 +90,9 @@ def rope_tables(dim: int, max_seq: int, theta: float = 500000.0,
                     "original_max_position_embeddings", 8192)))
         t = torch.arange(max_seq, dtype=torch.float64) / scaling
         freqs = torch.outer(t, inv_freq)
-        _table_cache[key] = (freqs.cos().float().to(device).contiguous(),
-                             freqs.sin().float().to(device).contiguous())
+        _table_cache[key] = (
+            (freqs.cos() * mag).float().to(device).contiguous(),
+            (freqs.sin() * mag).float().to(device).contiguous())
     return _table_cache[key]
 
 

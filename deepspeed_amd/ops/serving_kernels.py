@@ -27,6 +27,7 @@ COMMON = os.path.join(_SRC, "serving_common.h")
 #   rows   : norms, short convolutions, residual adds, activations, routers
 #   latent : compressed-KV attention
 #   seq    : windowed multi-head attention over paged K/V, linear recurrences
+#   recur  : gated diagonal recurrences
 LIBRARIES = {
     "rows": (os.path.join(_SRC, "serving_kernels.hip"),
              os.path.join(_HERE, "_serving.so")),
@@ -34,6 +35,8 @@ LIBRARIES = {
                os.path.join(_HERE, "_serving_latent.so")),
     "seq": (os.path.join(_SRC, "sequence_kernels.hip"),
             os.path.join(_HERE, "_serving_seq.so")),
+    "recur": (os.path.join(_SRC, "recurrence_kernels.hip"),
+              os.path.join(_HERE, "_serving_recur.so")),
 }
 SOURCE, LIBRARY = LIBRARIES["rows"]
 HIPCC_FLAGS = ["-O3", "-std=c++17", "--offload-arch=gfx950",
@@ -711,43 +714,67 @@ def _heads_view(t):
 def linear_scan(q, k, v, decay, beta, state, batch, q_scale=1.0):
     T, G, dim = q.shape
     H, vdim = v.shape[1], v.shape[2]
-    assert q.dtype == k.dtype == v.dtype and k.shape == q.shape
+    assert q.dtype == k.dtype and k.shape == q.shape
+    assert v.dtype == q.dtype or (q.dtype == torch.float32 and beta is None
+                                  and decay.dim() < 3)
     assert T == batch.n_tokens and v.shape[0] == T
     assert state.dtype == torch.float32 and state.is_contiguous()
     assert state.shape[1:] == (H, dim, vdim)
     assert decay.dtype == torch.float32 and decay.is_contiguous()
-    channel = decay.dim() == 3
-    assert decay.shape == ((T, H, dim) if channel else (T, H))
+    mode = {1: 2, 2: 0, 3: 1}[decay.dim()]      # fixed, per head, per channel
+    assert decay.shape == {2: (H,), 0: (T, H), 1: (T, H, dim)}[mode]
     if beta is not None:
         assert beta.shape == (T, H) and beta.dtype == torch.float32
         beta = beta.contiguous()
     out = torch.empty(T, H, vdim, dtype=torch.float32, device=q.device)
     (qp, ldq), (kp, ldk), (vp, ldv) = (_heads_view(t) for t in (q, k, v))
     _check(_seq().dsv_linear_scan(
-        qp, ldq, kp, ldk, vp, ldv, _p(decay), _i(1 if channel else 0),
+        qp, ldq, kp, ldk, vp, ldv, _p(decay), _i(mode),
         _p(beta), _p(state), _p(batch.cu), _p(batch.seq_slot), _p(out),
         _i(_dt(q)), _i(batch.n_seqs), _i(G), _i(H), _i(dim), _i(vdim),
-        _f(q_scale), _stream()), "linear_scan")
+        _f(q_scale), _i(_dt(v)), _stream()), "linear_scan")
     return out
 
 
-def head_norm_gate(o, weight, gate, eps, out_dtype, act="silu"):
+def head_norm_gate(o, weight, gate, eps, act, out_scale, out):
     T, H, vdim = o.shape
     assert o.dtype == torch.float32 and o.is_contiguous()
-    assert weight.numel() == vdim and gate.shape == (T, H * vdim)
-    assert gate.dtype == out_dtype
+    assert weight is None or weight.numel() == vdim
+    assert gate.shape == (T, H * vdim) == out.shape
+    assert gate.dtype == out.dtype
     _rows_ok(gate)
-    out = torch.empty(T, H * vdim, dtype=out_dtype, device=o.device)
+    _rows_ok(out)
     _check(_seq().dsv_head_norm_gate(
-        _p(o), _p(_f32(weight)), ctypes.c_void_p(gate.data_ptr()),
-        _i(gate.stride(0)), _p(out), _i(_DT[out_dtype]), _i(T), _i(H),
-        _i(vdim), _f(eps), _i(("silu", "sigmoid").index(act)), _stream()),
-        "head_norm_gate")
+        _p(o), _p(None if weight is None else _f32(weight).contiguous()),
+        _vp(gate), _i(gate.stride(0)), _vp(out), _i(out.stride(0)),
+        _i(_dt(out)), _i(T), _i(H), _i(vdim), _f(eps), _f(out_scale),
+        _i(("silu", "sigmoid").index(act)), _stream()), "head_norm_gate")
     return out
+
+
+def retention_prep(proj, batch, heads, dim, rot_dims, cos, sin, k_scale,
+                   layout):
+    T = proj.shape[0]
+    _rows_ok(proj)
+    assert T == batch.n_tokens and proj.shape[1] == 2 * heads * dim
+    assert rot_dims % 2 == 0 and rot_dims <= dim
+    if rot_dims:
+        assert cos.shape[1] == rot_dims // 2 and cos.shape[0] >= batch.max_ctx
+        assert cos.dtype == torch.float32 and sin.shape == cos.shape
+    q = torch.empty(T, heads, dim, dtype=torch.float32, device=proj.device)
+    k = torch.empty_like(q)
+    _check(_seq().dsv_retention_prep(
+        _vp(proj), _i(proj.stride(0)), _p(batch.tok_pos),
+        _p(cos if rot_dims else None), _p(sin if rot_dims else None), _p(q),
+        _p(k), _i(_dt(proj)), _i(T), _i(heads), _i(dim), _i(rot_dims),
+        _f(k_scale), _i(1 if layout == "half" else 0), _stream()),
+        "retention_prep")
+    return q, k
 
 
 # ------------------------------------- state-space prologues and epilogue
-def conv_silu_ragged(x, conv_w, state, batch, bias=None, out_dtype=None):
+def conv_silu_ragged(x, conv_w, state, batch, bias=None, out_dtype=None,
+                     act="silu"):
     T, C = x.shape
     taps = conv_w.shape[1]
     out_dtype = out_dtype or torch.float32
@@ -764,7 +791,8 @@ def conv_silu_ragged(x, conv_w, state, batch, bias=None, out_dtype=None):
         _l(state.stride(0)), _p(batch.cu), _p(batch.seq_slot),
         _p(batch.seq_start), _p(batch.tok_seq), _p(batch.tok_pos), _p(out),
         _i(_dt(x)), _i(0 if out_dtype == torch.float32 else 1), _i(T),
-        _i(batch.n_seqs), _i(C), _i(taps), _stream()), "conv_silu")
+        _i(batch.n_seqs), _i(C), _i(taps), _i(1 if act == "silu" else 0),
+        _stream()), "conv_silu")
     return out
 
 
@@ -924,6 +952,101 @@ def act_rows(z, act):
     out = torch.empty(T, F, dtype=z.dtype, device=z.device)
     _check(load().dsv_act_rows(_vp(z), _i(z.stride(0)), _p(out), _i(_dt(z)),
                                _l(T), _i(F), _i(act), _stream()), "act_rows")
+    return out
+
+
+def softcap_rows(z, cap):
+    z = z.contiguous()
+    out = torch.empty(z.shape, dtype=torch.float32, device=z.device)
+    _check(load().dsv_softcap_rows(_p(z), _p(out), _i(_dt(z)), _l(z.numel()),
+                                   _f(cap), _stream()), "softcap_rows")
+    return out
+
+
+# ------------------------------------------ pre-norm residual, token shift
+def residual_norm(x, y, mult, weight, bias, eps, out_dtype, extra, shift,
+                  state, batch, index):
+    T, C = x.shape
+    assert x.dtype == torch.float32 and x.is_contiguous()
+    assert weight.numel() == C and bias.numel() == C
+    if y is not None:
+        assert y.shape == x.shape
+        y = y.contiguous()
+    if extra is not None:
+        assert extra.numel() == C
+        extra = _f32(extra).contiguous()
+    adds = y is not None or extra is not None
+    rows, new = T, x
+    if index is not None:
+        index = index.to(torch.int64).contiguous()
+        rows = index.numel()
+    if shift is not None:
+        assert index is None and T == batch.n_tokens and shift.numel() == C
+        assert state.dtype == torch.float32 and state.is_contiguous()
+        assert state.shape[1:] == (C,)
+        if adds:
+            new = torch.empty_like(x)
+    h = torch.empty(rows, C, dtype=out_dtype, device=x.device)
+    b = batch if shift is not None else None
+    _check(load().dsv_residual_norm(
+        _p(x), _p(y), _i(0 if y is None else _dt(y)), _f(mult), _p(extra),
+        _p(_f32(weight).contiguous()), _p(_f32(bias).contiguous()),
+        _p(new if adds and index is None else None), _p(index),
+        _p(None if shift is None else _f32(shift).contiguous()),
+        _p(None if b is None else state), _p(b and b.cu),
+        _p(b and b.seq_slot), _p(b and b.seq_start), _p(b and b.tok_seq),
+        _p(h), _i(_DT[out_dtype]), _i(rows), _i(C), _f(eps), _stream()),
+        "residual_norm")
+    return new, h
+
+
+# ------------------------------------------------ gated diagonal recurrence
+def rglru_gates(u, w_r, b_r, w_i, b_i, lam, c, path=None):
+    """``path``: "mfma" (both block-diagonal products and the gates in one
+    kernel, bf16) or "split" (library products, then the gates; fp32)."""
+    T, W = u.shape
+    blocks, n, _ = w_r.shape
+    assert blocks * n == W and w_r.shape == w_i.shape == (blocks, n, n)
+    assert w_r.dtype == w_i.dtype == u.dtype and u.is_contiguous()
+    assert b_r.numel() == b_i.numel() == lam.numel() == W
+    a = torch.empty(T, W, dtype=torch.float32, device=u.device)
+    b = torch.empty_like(a)
+    lib = load("recur")
+    small = (_p(_f32(b_r).contiguous()), _p(_f32(b_i).contiguous()),
+             _p(_f32(lam).contiguous()))
+    if path is None:
+        path = "mfma" if u.dtype == torch.bfloat16 else "split"
+    if path == "mfma":
+        assert u.dtype == torch.bfloat16
+        _check(lib.dsv_rglru_gates(
+            _p(u), _p(w_r), _p(w_i), *small, _p(a), _p(b), _i(T), _i(blocks),
+            _i(n), _f(c), _stream()), "rglru_gates")
+        return a, b
+    ub = u.float().view(T, blocks, n).transpose(0, 1).contiguous()
+    zr = torch.bmm(ub, w_r.float().transpose(1, 2).contiguous())
+    zi = torch.bmm(ub, w_i.float().transpose(1, 2).contiguous())
+    _check(lib.dsv_rglru_pair(
+        _p(zr), _p(zi), _p(u), *small, _p(a), _p(b), _i(_dt(u)), _i(T),
+        _i(blocks), _i(n), _f(c), _stream()), "rglru_pair")
+    return a, b
+
+
+def diagonal_scan(a, b, state, batch, gate, act, out_dtype):
+    T, W = a.shape
+    assert a.is_contiguous() and b.is_contiguous() and b.shape == a.shape
+    assert a.dtype == b.dtype == state.dtype == torch.float32
+    assert T == batch.n_tokens and state.is_contiguous()
+    assert state.shape[1:] == (W,)
+    if gate is not None:
+        _rows_ok(gate)
+        assert gate.shape == (T, W) and gate.dtype == out_dtype
+    out = torch.empty(T, W, dtype=out_dtype, device=a.device)
+    _check(load("recur").dsv_diagonal_scan(
+        _p(a), _p(b), _p(None) if gate is None else _vp(gate),
+        _i(0 if gate is None else gate.stride(0)),
+        _i(("gelu_tanh", "silu").index(act)), _p(state), _p(batch.cu),
+        _p(batch.seq_slot), _p(out), _i(_dt(out)), _i(batch.n_seqs), _i(W),
+        _i(max(batch.counts)), _stream()), "diagonal_scan")
     return out
 
 

@@ -292,7 +292,7 @@ def test_three_band_frequencies():
 def test_rotation_layouts_and_scalings(layout, scaling):
     """attn_prep's rotation at scattered positions against the oracle; the
     coordinates beyond rot.dims pass unchanged."""
-    from deepspeed_amd.models.savovik import _rot_tables
+    from deepspeed_amd.models.savovik import rot_tables
     from deepspeed_amd.ops.window_attention import attn_prep
     torch.manual_seed(3)
     H, G, d, dv, dims = 2, 1, 10, 4, 6
@@ -302,7 +302,7 @@ def test_rotation_layouts_and_scalings(layout, scaling):
     held = 37
     cache, b = one_step_cache([G * (d + dv)], {}, [held], [5], tokens=64)
     proj = torch.randn(5, H * d + G * d + G * dv)
-    cos, sin = _rot_tables(rot, cache.max_seq, DEV)
+    cos, sin = rot_tables(rot, cache.max_seq, DEV)
     q = attn_prep(proj.to(DEV), b, cache.pools[0], None, None, 1e-6, H, G, d,
                   dv, dims, cos, sin, True, None, layout, None).cpu().double()
     want = O.rotate(proj[:, :H * d].double().reshape(5, H, d), rot, layout,

@@ -23,6 +23,12 @@ latent attention with sink and gate / two channel-decay delta layers, dense
 and routed feed-forwards with identity outputs) beside Lolulorn (the closest
 hybrid), Fizesun (the other latent-attention model) and Llama; every kernel on
 its path is timed next to the like kernel of those paths.
+
+``--serving redudra`` runs Redudra (gated diagonal recurrence / windowed
+attention beside retention, alternating, dense feed-forwards) beside Savovik
+(its closest sibling: parallel attention and recurrence on the ragged path),
+Lolulorn and Llama; every kernel on its path is timed next to the like kernel
+of those paths.
 """
 
 import json
@@ -1101,6 +1107,242 @@ def run_numolorn(sizes=("s", "m", "l"), kernels=True):
     return report
 
 
+# -------------------------------------------------------------- Redudra
+def redudra_config(z, vocab=32000):
+    """[gated diagonal recurrence, windowed attention beside retention]
+    alternating over ``layers``; attention heads of 128, 4 query heads per
+    key/value head, window 1024 + 4 kept tokens; retention heads with keys of
+    128 and values of 256 as Lolulorn's recurrent heads; recurrence as wide
+    as the model in blocks of 256; dense feed-forwards."""
+    W, H = z["width"], z["heads"]
+    RH = max(1, H // 2)
+    rg = {"width": W, "blocks": max(1, W // 256), "conv": 4}
+    par = {"left": {"heads": H, "kv_heads": max(1, H // 4), "dim": 128,
+                    "vdim": 128, "scale": 128 ** -0.5,
+                    "mask": {"size": 1024, "keep_first": 4},
+                    "rot": {"base": 10000.0, "dims": 128,
+                            "scaling": {"factor": 2.0, "original": 2048,
+                                        "fast": 32.0, "slow": 1.0}}},
+           "right": {"heads": RH, "dim": 128, "vdim": 256,
+                     "rot": {"base": 10000.0, "dims": 128},
+                     "decay": [1 - 2.0 ** -(5 + i % 8) for i in range(RH)]},
+           "left_scale": 1.0, "right_scale": 0.7}
+    ff = {"kind": "dense", "ff": z["ff"]}
+    layers = [{"type": "rglru" if i % 2 == 0 else "parallel",
+               "mixer": rg if i % 2 == 0 else par, "mlp": ff}
+              for i in range(z["layers"])]
+    return {"architecture": "Redudra", "vocab": vocab, "width": W,
+            "norm": {"eps": 1e-6}, "residual_mult": 0.5,
+            "logit_softcap": 30.0, "layers": layers}
+
+
+@torch.no_grad()
+def _redudra_kernel_rows(z, dev):
+    """Every kernel on Redudra's path at this size, each followed by the like
+    kernel of the Lolulorn or Savovik path at the same shapes ("like" names
+    it; rows with an empty "like" are the siblings themselves)."""
+    from ..ops import serving_kernels as sk
+    from ..ops.causal_conv import conv_silu_ragged
+    from ..ops.gated_recurrence import diagonal_scan, rglru_gates
+    from ..ops.linear_recurrence import (head_norm_gate, linear_scan,
+                                         retention_prep)
+    from ..ops.norms import residual_norm
+    from ..ops.rope import rope_tables
+    from .state_cache import PagedStateCache
+    bf = torch.bfloat16
+    B, S, W, H = z["batch"], z["seq"], z["width"], z["heads"]
+    F = z["ff"]
+    G, d, dv = max(1, H // 4), 128, 128
+    RH, rd, rv = max(1, H // 2), 128, 256
+    T = B * S
+    out = []
+
+    def row(name, like, fn, nbytes, flops=0.0, iters=5):
+        t = min(_timed(fn, 2, iters), _timed(fn, 1, iters))
+        bound = max(nbytes / HBM_BW, flops / MFMA_BF16)
+        out.append({"kernel": name, "like": like, "us": 1e6 * t,
+                    "bound_us": 1e6 * bound, "distance": t / bound})
+
+    # ---- residual add + norm (+ token shift) against the post-norm residual
+    cache = PagedStateCache([G * (d + dv)], {"shift": ((W,), torch.float32)},
+                            B, B * (S + 64), dtype=bf, device=dev)
+    batch = cache.begin_ragged(list(range(B)), [S] * B)
+    x32 = torch.randn(T, W, device=dev)
+    y1 = (torch.randn(T, W, device=dev) * 0.01).to(bf)
+    wn, bn = torch.ones(W, device=dev), torch.zeros(W, device=dev)
+    mu = torch.full((W,), 0.5, device=dev)
+    row("residual_norm with token shift (fp32 stream += m * bf16, bf16 out)",
+        "layer_norm_add",
+        lambda: residual_norm(x32, y1, 0.5, wn, bn, 1e-6, bf, None, mu,
+                              cache.states["shift"], batch), T * W * 12)
+    row("residual_norm (fp32 stream += m * bf16, bf16 norm out)",
+        "layer_norm_add",
+        lambda: residual_norm(x32, y1, 0.5, wn, bn, 1e-6, bf), T * W * 12)
+    row("layer_norm_add (lolulorn)", "",
+        lambda: sk.layer_norm_add(x32, y1, wn, bn, 1e-6, bf), T * W * 12)
+    # ---- prologues
+    cos, sin = rope_tables(d, cache.max_seq, 10000.0, device=dev)
+    proj = torch.randn(T, (H + 2 * G) * d, device=dev).to(bf)
+    nb = T * (H + 2 * G) * d * 4
+    row("attn_prep: rotate-half, no norms, cache write", "attn_prep",
+        lambda: sk.attn_prep(proj, batch, cache.pools[0], None, None, 1e-6, H,
+                             G, d, dv, d, cos, sin, True, None, "half",
+                             None), nb)
+    qk = torch.randn(T, 2 * RH * rd, device=dev).to(bf)
+    row("retention_prep: rotate-half, scaled keys, fp32 out", "attn_prep",
+        lambda: retention_prep(qk, batch, RH, rd, rd, cos, sin, rd ** -0.5),
+        T * 2 * RH * rd * 6)
+    qw, kw = torch.ones(H * d, device=dev), torch.ones(G * d, device=dev)
+    row("attn_prep (lolulorn: whole-projection norms)", "",
+        lambda: sk.attn_prep(proj, batch, cache.pools[0], qw, kw, 1e-6, H, G,
+                             d, dv, d, cos, sin, True), nb)
+    # ---- prefill attention (the kernel is the same one)
+    q = sk.attn_prep(proj, batch, cache.pools[0], None, None, 1e-6, H, G, d,
+                     dv, d, cos, sin, True, None, "half", None)
+    win = 1024
+    seen = sum(min(i + 1, win) + min(4, max(0, i + 1 - win))
+               for i in range(S))
+    both = torch.empty(T, H * dv + RH * rv, device=dev, dtype=bf)
+    io = T * H * (d + dv) * 2 + T * G * (d + dv) * 2
+    row("window_attention prefill (window + kept, into a wider row)",
+        "window_attention prefill",
+        lambda: sk.window_attention(q, cache.pools[0], batch, G, d, dv,
+                                    d ** -0.5, win, 4, None, 0, 0.0, 1.2,
+                                    both[:, :H * dv]),
+        io, 2.0 * B * H * seen * (d + dv), iters=2)
+    row("window_attention prefill (lolulorn: window %d + 4 kept)" % win, "",
+        lambda: sk.window_attention(q, cache.pools[0], batch, G, d, dv,
+                                    d ** -0.5, win, 4),
+        io, 2.0 * B * H * seen * (d + dv), iters=2)
+    cache.end_step()
+    del proj, q
+    for NB in (B, 64):
+        big = PagedStateCache([G * (d + dv)], {}, NB, NB * (S + 64), dtype=bf,
+                              device=dev)
+        big.pools[0].normal_()
+        for i in range(NB):
+            big.lens[i] = S
+        bt = big.begin_ragged(list(range(NB)), [1] * NB)
+        qd = (torch.randn(NB, H, d, device=dev) * 0.1).to(bf)
+        wide = torch.empty(NB, H * dv + RH * rv, device=dev, dtype=bf)
+        nbytes = NB * min(S + 1, win + 4) * G * (d + dv) * 2
+        row("window_attention decode (into a wider row), %d requests" % NB,
+            "window_attention decode",
+            lambda: sk.window_attention(qd, big.pools[0], bt, G, d, dv,
+                                        d ** -0.5, win, 4, None, 0, 0.0, 1.2,
+                                        wide[:, :H * dv]), nbytes)
+        row("window_attention decode (lolulorn), %d requests" % NB, "",
+            lambda: sk.window_attention(qd, big.pools[0], bt, G, d, dv,
+                                        d ** -0.5, win, 4), nbytes)
+        big.end_step()
+        del big
+    # ---- matrix-state recurrence: fixed decay beside a decay per channel
+    for NB, cnt in ((B, S), (B, 1), (64, 1)):
+        rc = PagedStateCache([], {"rec": ((RH, rd, rv), torch.float32)}, NB,
+                             NB * (S + 64), dtype=bf, device=dev)
+        bt = rc.begin_ragged(list(range(NB)), [cnt] * NB)
+        n = NB * cnt
+        st = rc.states["rec"]
+        qq = torch.randn(n, RH, rd, device=dev) * 0.1
+        kk = torch.randn(n, RH, rd, device=dev) * 0.1
+        vv = torch.randn(n, RH, rv, device=dev).to(bf)
+        dec = torch.full((RH,), 0.99, device=dev)
+        io = n * RH * (2 * rd + rv) * 2 + n * RH * rv * 4 \
+            + 2 * NB * RH * rd * rv * 4
+        fl = n * RH * 4.0 * rd * rv
+        row("linear_scan retention, %d x %d tokens" % (NB, cnt),
+            "linear_scan gla",
+            lambda: linear_scan(qq, kk, vv, dec, None, st, bt),
+            io + n * RH * 2 * rd * 2, fl)
+        q16, k16 = qq.to(bf), kk.to(bf)
+        dch = torch.rand(n, RH, rd, device=dev) * 0.1 + 0.9
+        row("linear_scan gla (lolulorn), %d x %d tokens" % (NB, cnt), "",
+            lambda: linear_scan(q16, k16, vv, dch, None, st, bt),
+            io + n * RH * rd * 4, fl)
+        rc.end_step()
+        del rc, qq, kk, vv, dch, q16, k16
+    o32 = torch.randn(T, RH, rv, device=dev)
+    gate = torch.randn(T, RH * rv, device=dev).to(bf)
+    nw = torch.ones(rv, device=dev)
+    row("head_norm_gate (no weight, scaled, into a wider row)",
+        "head_norm_gate",
+        lambda: head_norm_gate(o32, None, gate, 1e-6, bf, "silu", 0.5,
+                               both[:, H * dv:]), T * RH * rv * 8)
+    row("head_norm_gate (lolulorn)", "",
+        lambda: head_norm_gate(o32, nw, gate, 1e-6, bf), T * RH * rv * 8)
+    del o32, gate, both
+    # ---- gated diagonal recurrence against the selective scan
+    nbk = max(1, W // 256)
+    wr = (torch.randn(nbk, W // nbk, W // nbk, device=dev) * 0.06).to(bf)
+    wi = (torch.randn(nbk, W // nbk, W // nbk, device=dev) * 0.06).to(bf)
+    zero = torch.zeros(W, device=dev)
+    cw = torch.randn(W, 4, device=dev).to(bf)
+    SN = 16
+    a_log = torch.zeros(W, SN, device=dev)
+    for NB, cnt in ((B, S), (B, 1), (64, 1)):
+        n = NB * cnt
+        case = "%d x %d tokens" % (NB, cnt)
+        rc = PagedStateCache([], {"conv": (3, W), "rec": ((W,),
+                                                          torch.float32),
+                                  "sel": ((W, SN), torch.float32)}, NB,
+                             NB * (S + 64), dtype=bf, device=dev)
+        bt = rc.begin_ragged(list(range(NB)), [cnt] * NB)
+        pin = torch.randn(n, 2 * W, device=dev).to(bf)
+        row("conv (bias, no activation), " + case, "conv_silu",
+            lambda: conv_silu_ragged(pin[:, W:], cw, rc.states["conv"], bt,
+                                     zero, bf, None), n * W * 4)
+        row("conv_silu (savovik), " + case, "",
+            lambda: conv_silu_ragged(pin[:, W:], cw, rc.states["conv"], bt,
+                                     zero, bf), n * W * 4)
+        u = torch.randn(n, W, device=dev).to(bf)
+        row("rglru_gates (both block products, gates), " + case,
+            "sigmoid_pow",
+            lambda: rglru_gates(u, wr, zero, wi, zero, zero),
+            n * W * 10 + 4 * W * (W // nbk), 4.0 * n * W * (W // nbk))
+        row("sigmoid_pow (lolulorn: bf16 in, fp32 out), " + case, "",
+            lambda: sk.sigmoid_pow(u, zero, 1.0 / 16), n * W * 6)
+        a, bb = rglru_gates(u, wr, zero, wi, zero, zero)
+        row("diagonal_scan (gated read-out), " + case, "selective_scan",
+            lambda: diagonal_scan(a, bb, rc.states["rec"], bt, pin[:, :W],
+                                  "gelu_tanh", bf),
+            n * W * 12 + 2 * NB * W * 4)
+        bc = (torch.randn(n, 2 * SN, device=dev) * 0.1).to(bf)
+        so = torch.empty(n, W, device=dev, dtype=bf)
+        row("selective_scan (savovik), " + case, "",
+            lambda: sk.selective_scan(u, a, zero, a_log, bc[:, :SN],
+                                      bc[:, SN:], zero, pin[:, :W],
+                                      rc.states["sel"], bt, 1.0, so),
+            n * W * 10 + n * 2 * SN * 2 + 2 * NB * W * SN * 4)
+        rc.end_step()
+        del rc, pin, u, a, bb
+    gu = torch.randn(T, 2 * F, device=dev).to(bf)
+    row("glu silu (also lolulorn's)", "", lambda: sk.glu(gu, 0), T * F * 6)
+    lg = torch.randn(64, 32000, device=dev).to(bf)
+    row("softcap_rows, 64 x 32000", "",
+        lambda: sk.softcap_rows(lg, 30.0), 64 * 32000 * 6)
+    return out
+
+
+def run_redudra(sizes=("s", "m", "l"), kernels=True):
+    dev = torch.device("cuda", torch.cuda.current_device())
+    report = {}
+    for name in sizes:
+        z = dict(SIZES[name])
+        z["layers"] = 4
+        rec = {"size": {k: z[k] for k in z},
+               "redudra": _ragged_throughput(redudra_config(z), z, dev),
+               "savovik": _ragged_throughput(savovik_config(z), z, dev),
+               "lolulorn": _ragged_throughput(lolulorn_config(z), z, dev),
+               "llama": _llama_throughput(z, dev)}
+        if kernels:
+            rows = _redudra_kernel_rows(z, dev)
+            rec["kernels"] = rows
+            rec["distance_over_sibling"] = _sibling_ratios(rows)
+        report[name] = rec
+        torch.cuda.empty_cache()
+    return report
+
+
 def _same_case(a, b):
     """Rows of one case carry the same '<n> requests' / '<n> x <m> tokens'."""
     import re
@@ -1124,6 +1366,24 @@ def run(sizes=("s", "m", "l"), kernels=True):
 
 def main(sizes="s,m,l", out=None, model="fizesun"):
     names = tuple(sizes.split(","))
+    if model == "redudra":
+        rep = run_redudra(names)
+        if out:
+            with open(out, "w") as f:
+                json.dump(rep, f, indent=1)
+        best = rep[names[-1]]
+        print(json.dumps({
+            "metric": "redudra_serving_tokens_per_s", "unit": "tokens/s",
+            "dtype": "bf16", "data": "synthetic", "n_gpus": 1,
+            "value": best["redudra"]["prefill_tok_s"],
+            "higher_is_better": True,
+            "sizes": {k: {"redudra": v["redudra"], "savovik": v["savovik"],
+                          "lolulorn": v["lolulorn"], "llama": v["llama"],
+                          "worst_distance_over_sibling": max(
+                              v.get("distance_over_sibling", {}).values(),
+                              default=None)}
+                      for k, v in rep.items()}}))
+        return rep
     if model == "numolorn":
         rep = run_numolorn(names)
         if out:

@@ -1,6 +1,7 @@
-// Gated diagonal recurrences over ragged batches for MI355X (gfx950): the
-// block-diagonal gates of a real-gated linear recurrent unit and the scan of
-// a recurrence with one state per channel.
+// Recurrences over ragged batches for MI355X (gfx950): the block-diagonal
+// gates of a real-gated linear recurrent unit, the scan of a recurrence with
+// one state per channel, and the chunked form of a matrix-state recurrence
+// with one fixed decay per head.
 //
 // Plain C ABI (raw device pointers + a hipStream_t) so the library builds in
 // seconds with hipcc alone and is loaded through ctypes. dtype codes:
@@ -304,6 +305,345 @@ __global__ __launch_bounds__(NT) void diagonal_scan_short_k(
   *Sg = S;
 }
 
+// ------------------------- matrix-state recurrence with a fixed decay, chunks
+// S <- g S + k v^T, o = S^T q per head, RC tokens at a time on matrix cores:
+// with a chunk's tokens 0..n-1 and the state S0 before it,
+//   o_t = g^(t+1) S0^T q_t + sum_{s<=t} g^(t-s) (q_t . k_s) v_s
+//   S   = g^n S0 + sum_s (g^(n-1-s) k_s) v_s^T.
+// q and k are float, v bf16. Every float operand of a product (q, k, the
+// decayed keys, the masked scores, the state) enters as a bf16 head plus a
+// bf16 remainder, i.e. with 16 bits of mantissa, and the product of the two
+// remainders is dropped; sums and the state itself (accumulators, RN columns
+// of one head per workgroup, kept over all chunks) are float.
+//
+// 4 waves: wave w owns tokens 16w..16w+15 of the chunk and rows
+// w*DP/4..(w+1)*DP/4-1 of the state. LDS holds the keys by token, the decayed
+// keys and the values by coordinate (token-contiguous) and the state by value
+// column; rows are split into 16-byte groups whose order is permuted by the
+// row, which spreads both the writes (rows 4i + e over lanes i) and the reads
+// (16 neighbouring rows) over the banks. The scores are made transposed (keys
+// as rows), so that a lane's accumulators are four neighbouring keys of its
+// own token: they are the A operand of the product with v as they are, with
+// the key order of both operands permuted alike. The next chunk's q, k, v are
+// in flight while a chunk is computed.
+typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
+typedef __attribute__((ext_vector_type(4))) __bf16 bf16x4;
+constexpr int RC = 64;  // tokens per chunk
+constexpr int RN = 64;  // value columns per workgroup
+
+// offset of element (row, col) in rows of `pitch` elements (whole 64s)
+__device__ __forceinline__ int swz(int row, int col, int pitch) {
+  return row * pitch + (((col >> 3) ^ ((row ^ (row >> 2)) & 7)) << 3) + (col & 7);
+}
+__device__ __forceinline__ void split2(float x, __bf16& hi, __bf16& lo) {
+  hi = static_cast<__bf16>(x);
+  lo = static_cast<__bf16>(x - static_cast<float>(hi));
+}
+__device__ __forceinline__ floatx4 mma(bf16x8 a, bf16x8 b, floatx4 c) {
+  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0);
+}
+
+template <int DP>
+__global__ __launch_bounds__(256) void retention_chunk_k(
+    const float* __restrict__ q, const float* __restrict__ k, const bf16* __restrict__ v,
+    int ld_v, const float* __restrict__ decay, float* __restrict__ state,
+    const int* __restrict__ cu, const int* __restrict__ seq_slot, float* __restrict__ out, int G,
+    int H, int dim, int vdim, float q_scale) {
+  constexpr int KS = DP / 32;   // 32-wide steps over a head's coordinates
+  constexpr int MT = DP / 64;   // 16-row tiles of the state per wave
+  constexpr int NT4 = RN / 16;  // 16-column tiles
+  constexpr int KQ = DP / 4;    // groups of four coordinates
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  __bf16* Kh = reinterpret_cast<__bf16*>(smem);  // [RC][DP]
+  __bf16* Kl = Kh + RC * DP;
+  __bf16* Dh = Kl + RC * DP;  // [DP][RC] keys times their decay to the chunk's end
+  __bf16* Dl = Dh + DP * RC;
+  __bf16* Sh = Dl + DP * RC;  // [RN][DP]
+  __bf16* Sl = Sh + RN * DP;
+  __bf16* Vt = Sl + RN * DP;  // [RN][RC]
+  const int s = blockIdx.x, h = blockIdx.y, c0 = blockIdx.z * RN;
+  const int t0 = cu[s], cnt = cu[s + 1] - t0;
+  if (cnt <= 0) return;  // whole workgroup
+  const int g = h / (H / G);
+  const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
+  const int l15 = lane & 15, quad = lane >> 4;
+  const float lg = fmaxf(log2f(decay[h]), -1000.f);
+  auto pw = [&](int e) { return __builtin_amdgcn_exp2f(lg * (float)e); };
+  const int ldq = G * dim;
+  const float* qb = q + (int64_t)t0 * ldq + g * dim;
+  const float* kb = k + (int64_t)t0 * ldq + g * dim;
+  const bf16* vb = v + (int64_t)t0 * ld_v + h * vdim + c0;
+
+  // this lane's part of the state, accumulator layout: row (coordinate)
+  // w*DP/4 + 16 mt + 4 quad + j, column c0 + 16 nt + l15
+  float* Sg = state + (((int64_t)seq_slot[s] * H + h) * dim) * vdim + c0;
+  floatx4 S[MT][NT4];
+#pragma unroll
+  for (int mt = 0; mt < MT; ++mt)
+#pragma unroll
+    for (int nt = 0; nt < NT4; ++nt)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int d = w * (DP / 4) + mt * 16 + quad * 4 + j, c = nt * 16 + l15;
+        S[mt][nt][j] = d < dim && c0 + c < vdim ? Sg[(int64_t)d * vdim + c] : 0.f;
+      }
+
+  // staging: a thread moves four coordinates of eight tokens of k, and four
+  // columns of eight tokens of v; of q a lane holds its token's A operands
+  const int kq = threadIdx.x % KQ, kg = threadIdx.x / KQ;
+  const bool kin = kg < RC / 8;
+  const int vq = (threadIdx.x - 128) & 15, vg = (threadIdx.x - 128) >> 4;
+  const bool vin = threadIdx.x >= 128;
+  float4 rk[8], rq[KS][2];
+  uint2 rv[8];
+  auto fetch = [&](int base) {
+    const int n = min(RC, cnt - base);
+    const float4 z4 = make_float4(0.f, 0.f, 0.f, 0.f);
+    if (kin) {
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        const int t = kg * 8 + i;
+        rk[i] = t < n && kq * 4 < dim
+                    ? *reinterpret_cast<const float4*>(kb + (int64_t)(base + t) * ldq + kq * 4)
+                    : z4;
+      }
+    }
+    if (vin) {
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        const int t = vg * 8 + i;
+        rv[i] = t < n && c0 + vq * 4 < vdim
+                    ? *reinterpret_cast<const uint2*>(vb + (int64_t)(base + t) * ld_v + vq * 4)
+                    : make_uint2(0u, 0u);
+      }
+    }
+    const int t = w * 16 + l15;
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks)
+#pragma unroll
+      for (int e = 0; e < 2; ++e) {
+        const int d = ks * 32 + quad * 8 + e * 4;
+        rq[ks][e] = t < n && d < dim
+                        ? *reinterpret_cast<const float4*>(qb + (int64_t)(base + t) * ldq + d)
+                        : z4;
+      }
+  };
+  auto stash = [&](int n) {
+    if (kin) {
+      float f[8];
+#pragma unroll
+      for (int i = 0; i < 8; ++i) f[i] = pw(max(n - 1 - (kg * 8 + i), 0));
+      bf16x8 th[4], tl[4];
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        const float x[4] = {rk[i].x, rk[i].y, rk[i].z, rk[i].w};
+        bf16x4 hi, lo;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          __bf16 a, b;
+          split2(x[e], a, b);
+          hi[e] = a;
+          lo[e] = b;
+          split2(x[e] * f[i], a, b);
+          th[e][i] = a;
+          tl[e][i] = b;
+        }
+        const int at = swz(kg * 8 + i, kq * 4, DP);
+        *reinterpret_cast<bf16x4*>(Kh + at) = hi;
+        *reinterpret_cast<bf16x4*>(Kl + at) = lo;
+      }
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const int at = swz(kq * 4 + e, kg * 8, RC);
+        *reinterpret_cast<bf16x8*>(Dh + at) = th[e];
+        *reinterpret_cast<bf16x8*>(Dl + at) = tl[e];
+      }
+    }
+    if (vin) {
+      bf16x8 tv[4];
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        const bf16x4 x = __builtin_bit_cast(bf16x4, rv[i]);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) tv[e][i] = x[e];
+      }
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+        *reinterpret_cast<bf16x8*>(Vt + swz(vq * 4 + e, vg * 8, RC)) = tv[e];
+    }
+#pragma unroll
+    for (int mt = 0; mt < MT; ++mt)
+#pragma unroll
+      for (int nt = 0; nt < NT4; ++nt) {
+        bf16x4 hi, lo;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          __bf16 a, b;
+          split2(S[mt][nt][j], a, b);
+          hi[j] = a;
+          lo[j] = b;
+        }
+        const int at = swz(nt * 16 + l15, w * (DP / 4) + mt * 16 + quad * 4, DP);
+        *reinterpret_cast<bf16x4*>(Sh + at) = hi;
+        *reinterpret_cast<bf16x4*>(Sl + at) = lo;
+      }
+  };
+
+  fetch(0);
+  for (int base = 0; base < cnt; base += RC) {
+    const int n = min(RC, cnt - base);
+    stash(n);
+    bf16x8 qh[KS], ql[KS];
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) {
+      const float x[8] = {rq[ks][0].x, rq[ks][0].y, rq[ks][0].z, rq[ks][0].w,
+                          rq[ks][1].x, rq[ks][1].y, rq[ks][1].z, rq[ks][1].w};
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        __bf16 a, b;
+        split2(x[e] * q_scale, a, b);
+        qh[ks][e] = a;
+        ql[ks][e] = b;
+      }
+    }
+    __syncthreads();
+    if (base + RC < cnt) fetch(base + RC);
+
+    // masked, decayed scores: p[jt][j] for key 16 jt + 4 quad + j, token l15
+    floatx4 p[4];
+#pragma unroll
+    for (int jt = 0; jt < 4; ++jt) {
+      floatx4 acc = {0.f, 0.f, 0.f, 0.f};
+      if (jt <= w) {
+#pragma unroll
+        for (int ks = 0; ks < KS; ++ks) {
+          const int at = swz(jt * 16 + l15, ks * 32 + quad * 8, DP);
+          const bf16x8 kh = *reinterpret_cast<const bf16x8*>(Kh + at);
+          const bf16x8 kl = *reinterpret_cast<const bf16x8*>(Kl + at);
+          acc = mma(kh, qh[ks], acc);
+          acc = mma(kl, qh[ks], acc);
+          acc = mma(kh, ql[ks], acc);
+        }
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          const int dt = (w - jt) * 16 + l15 - quad * 4 - j;
+          acc[j] = dt >= 0 ? acc[j] * pw(dt) : 0.f;
+        }
+      }
+      p[jt] = acc;
+    }
+    // what the earlier chunks' state gives, then this chunk's own tokens
+    floatx4 o[NT4];
+#pragma unroll
+    for (int nt = 0; nt < NT4; ++nt) {
+      o[nt] = (floatx4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int ks = 0; ks < KS; ++ks) {
+        const int at = swz(nt * 16 + l15, ks * 32 + quad * 8, DP);
+        const bf16x8 sh = *reinterpret_cast<const bf16x8*>(Sh + at);
+        const bf16x8 sl = *reinterpret_cast<const bf16x8*>(Sl + at);
+        o[nt] = mma(qh[ks], sh, o[nt]);
+        o[nt] = mma(ql[ks], sh, o[nt]);
+        o[nt] = mma(qh[ks], sl, o[nt]);
+      }
+    }
+    float f[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) f[j] = pw(w * 16 + quad * 4 + j + 1);
+#pragma unroll
+    for (int nt = 0; nt < NT4; ++nt)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) o[nt][j] *= f[j];
+#pragma unroll
+    for (int kp = 0; kp < 2; ++kp) {
+      if (2 * kp > w) continue;  // wave-uniform
+      bf16x8 ph, pl;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        __bf16 a, b;
+        split2(p[2 * kp + (e >> 2)][e & 3], a, b);
+        ph[e] = a;
+        pl[e] = b;
+      }
+#pragma unroll
+      for (int nt = 0; nt < NT4; ++nt) {
+        const int r = nt * 16 + l15;
+        const bf16x4 a =
+            *reinterpret_cast<const bf16x4*>(Vt + swz(r, (2 * kp) * 16 + quad * 4, RC));
+        const bf16x4 b =
+            *reinterpret_cast<const bf16x4*>(Vt + swz(r, (2 * kp + 1) * 16 + quad * 4, RC));
+        const bf16x8 vf = __builtin_shufflevector(a, b, 0, 1, 2, 3, 4, 5, 6, 7);
+        o[nt] = mma(ph, vf, o[nt]);
+        o[nt] = mma(pl, vf, o[nt]);
+      }
+    }
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const int t = w * 16 + quad * 4 + j;
+      if (t < n) {
+        float* row = out + ((int64_t)(t0 + base + t) * H + h) * vdim + c0;
+#pragma unroll
+        for (int nt = 0; nt < NT4; ++nt)
+          if (c0 + nt * 16 + l15 < vdim) row[nt * 16 + l15] = o[nt][j];
+      }
+    }
+    // the state after the chunk
+    const float gn = pw(n);
+#pragma unroll
+    for (int mt = 0; mt < MT; ++mt)
+#pragma unroll
+      for (int nt = 0; nt < NT4; ++nt)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) S[mt][nt][j] *= gn;
+#pragma unroll
+    for (int kk = 0; kk < 2; ++kk) {
+      bf16x8 vf[NT4];
+#pragma unroll
+      for (int nt = 0; nt < NT4; ++nt)
+        vf[nt] = *reinterpret_cast<const bf16x8*>(
+            Vt + swz(nt * 16 + l15, kk * 32 + quad * 8, RC));
+#pragma unroll
+      for (int mt = 0; mt < MT; ++mt) {
+        const int at = swz(w * (DP / 4) + mt * 16 + l15, kk * 32 + quad * 8, RC);
+        const bf16x8 dh = *reinterpret_cast<const bf16x8*>(Dh + at);
+        const bf16x8 dl = *reinterpret_cast<const bf16x8*>(Dl + at);
+#pragma unroll
+        for (int nt = 0; nt < NT4; ++nt) {
+          S[mt][nt] = mma(dh, vf[nt], S[mt][nt]);
+          S[mt][nt] = mma(dl, vf[nt], S[mt][nt]);
+        }
+      }
+    }
+    __syncthreads();  // every read of this chunk's LDS is done
+  }
+#pragma unroll
+  for (int mt = 0; mt < MT; ++mt)
+#pragma unroll
+    for (int nt = 0; nt < NT4; ++nt)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int d = w * (DP / 4) + mt * 16 + quad * 4 + j, c = nt * 16 + l15;
+        if (d < dim && c0 + c < vdim) Sg[(int64_t)d * vdim + c] = S[mt][nt][j];
+      }
+}
+
+template <int DP>
+int launch_retention_chunk(const float* q, const float* k, const void* v, int ld_v,
+                           const float* decay, float* state, const int* cu, const int* seq_slot,
+                           float* out, int nseq, int G, int H, int dim, int vdim, float q_scale,
+                           hipStream_t s) {
+  const int lds = (4 * RC * DP + 2 * RN * DP + RN * RC) * 2;
+  auto kern = retention_chunk_k<DP>;
+  if (lds > 48 * 1024) {
+    hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kern),
+                                       hipFuncAttributeMaxDynamicSharedMemorySize, lds);
+    if (e != hipSuccess) return (int)e;
+  }
+  kern<<<dim3(nseq, H, (vdim + RN - 1) / RN), 256, lds, s>>>(
+      q, k, (const bf16*)v, ld_v, decay, state, cu, seq_slot, out, G, H, dim, vdim, q_scale);
+  return (int)hipGetLastError();
+}
+
 }  // namespace
 
 extern "C" {
@@ -357,6 +697,27 @@ int dsv_diagonal_scan(const float* a, const float* b, const void* gate, int ld_g
     BY_DTYPE(dt, (diagonal_scan_k<T, 32><<<dim3(nseq, (W + 31) / 32), DS_T, 0, s>>>(
                      a, b, (const T*)gate, ld_gate, act, state, cu, seq_slot, (T*)out, W)));
   return (int)hipGetLastError();
+}
+
+// largest head size of keys the chunked form covers
+int dsv_retention_chunk_max_dim() { return 128; }
+
+// float q, k [T, G*dim] (contiguous), bf16 v (row stride ld_v), decay [H];
+// dim, vdim and ld_v multiples of 4, q and k 16-byte and v 8-byte aligned
+int dsv_retention_chunk(const float* q, const float* k, const void* v, int ld_v,
+                        const float* decay, float* state, const int* cu, const int* seq_slot,
+                        float* out, int nseq, int G, int H, int dim, int vdim, float q_scale,
+                        hipStream_t s) {
+  if (dim < 1 || dim > dsv_retention_chunk_max_dim() || vdim < 1 || G < 1 || H % G) return -1;
+  if (dim % 4 || vdim % 4 || ld_v % 4 || (uintptr_t)q % 16 || (uintptr_t)k % 16 ||
+      (uintptr_t)v % 8)
+    return -2;
+  if (nseq <= 0) return 0;
+  if (dim <= 64)
+    return launch_retention_chunk<64>(q, k, v, ld_v, decay, state, cu, seq_slot, out, nseq, G, H,
+                                      dim, vdim, q_scale, s);
+  return launch_retention_chunk<128>(q, k, v, ld_v, decay, state, cu, seq_slot, out, nseq, G, H,
+                                     dim, vdim, q_scale, s);
 }
 
 }  // extern "C"

@@ -27,7 +27,7 @@ COMMON = os.path.join(_SRC, "serving_common.h")
 #   rows   : norms, short convolutions, residual adds, activations, routers
 #   latent : compressed-KV attention
 #   seq    : windowed multi-head attention over paged K/V, linear recurrences
-#   recur  : gated diagonal recurrences
+#   recur  : gated diagonal recurrences, chunked fixed-decay recurrence
 LIBRARIES = {
     "rows": (os.path.join(_SRC, "serving_kernels.hip"),
              os.path.join(_HERE, "_serving.so")),
@@ -711,7 +711,13 @@ def _heads_view(t):
     return ctypes.c_void_p(t.data_ptr()), _i(t.stride(0))
 
 
-def linear_scan(q, k, v, decay, beta, state, batch, q_scale=1.0):
+CHUNK_MIN = 16      # fewer tokens per sequence: the token-by-token scan
+
+
+def linear_scan(q, k, v, decay, beta, state, batch, q_scale=1.0, path=None):
+    """``path`` forces "scan" (token by token) or "chunk" (matrix cores: fixed
+    decay per head, fp32 q and k with 16-bit v); default: chunks for prompt
+    portions where they apply."""
     T, G, dim = q.shape
     H, vdim = v.shape[1], v.shape[2]
     assert q.dtype == k.dtype and k.shape == q.shape
@@ -728,6 +734,21 @@ def linear_scan(q, k, v, decay, beta, state, batch, q_scale=1.0):
         beta = beta.contiguous()
     out = torch.empty(T, H, vdim, dtype=torch.float32, device=q.device)
     (qp, ldq), (kp, ldk), (vp, ldv) = (_heads_view(t) for t in (q, k, v))
+    chunked = mode == 2 and beta is None and q.dtype == torch.float32 \
+        and v.dtype == torch.bfloat16 and q.is_contiguous() \
+        and k.is_contiguous() and dim % 4 == 0 and vdim % 4 == 0 \
+        and v.stride(0) % 4 == 0 and v.data_ptr() % 8 == 0 \
+        and dim <= load("recur").dsv_retention_chunk_max_dim()
+    if path is None:
+        path = "chunk" if chunked and max(batch.counts) >= CHUNK_MIN \
+            else "scan"
+    if path == "chunk":
+        assert chunked, "operands the chunked form does not cover"
+        _check(load("recur").dsv_retention_chunk(
+            qp, kp, vp, ldv, _p(decay), _p(state), _p(batch.cu),
+            _p(batch.seq_slot), _p(out), _i(batch.n_seqs), _i(G), _i(H),
+            _i(dim), _i(vdim), _f(q_scale), _stream()), "linear_scan(chunk)")
+        return out
     _check(_seq().dsv_linear_scan(
         qp, ldq, kp, ldk, vp, ldv, _p(decay), _i(mode),
         _p(beta), _p(state), _p(batch.cu), _p(batch.seq_slot), _p(out),

@@ -1130,6 +1130,42 @@ def test_scan_with_a_fixed_decay_against_eager(H, d, dv, vdt, monkeypatch):
 
 
 @pytest.mark.gpu
+@pytest.mark.parametrize("counts", [[1, 70, 20], [64, 63, 65], [2, 200, 128],
+                                    [16]])
+@pytest.mark.parametrize("H,G,d,dv", [(3, 3, 8, 4), (2, 2, 64, 64),
+                                      (4, 2, 128, 48), (1, 1, 100, 260),
+                                      (2, 1, 36, 128)])
+def test_chunked_scan_against_the_token_by_token_scan(H, G, d, dv, counts,
+                                                      monkeypatch):
+    """Portions at, around and far from a chunk's length, decays from one that
+    forgets at once to one that never does, states that hold something."""
+    from deepspeed_amd.ops import serving_kernels as sk
+    from deepspeed_amd.ops.linear_recurrence import linear_scan
+    T, n = sum(counts), len(counts)
+    q, k = rnd(T, G, d).to(DEV), (rnd(T, G, d, seed=1) * d ** -0.5).to(DEV)
+    v = rnd(T, H * dv + 8, seed=2).to(DEV, torch.bfloat16)[:, 4:4 + H * dv] \
+        .view(T, H, dv)
+    dec = torch.tensor([0.99, 1.0, 0.0, 0.3][:H]).to(DEV)
+    st0 = rnd(n, H, d, dv, seed=3).to(DEV)
+
+    def run(path):
+        _, bt = begun({}, [3] * n, counts)
+        st = st0.clone()
+        return sk.linear_scan(q, k, v, dec, None, st, bt, 0.7, path), st
+
+    got, want = run("chunk"), run("scan")
+    for g, e in zip(got, want):
+        err = (g - e).abs().max() / e.abs().max()
+        assert err < 5e-5, "relative error %.3g" % err
+    monkeypatch.setenv("DS_AMD_SERVING_EAGER", "1")
+    _, bt = begun({}, [3] * n, counts)
+    st = st0.clone()
+    near(want[0], linear_scan(q, k, v, dec, None, st, bt, 0.7),
+         torch.float32)
+    near(want[1], st, torch.float32)
+
+
+@pytest.mark.gpu
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 @pytest.mark.parametrize("H,v,weight,act", [
     (3, 5, True, "silu"), (4, 64, False, "silu"), (3, 128, True, "sigmoid"),

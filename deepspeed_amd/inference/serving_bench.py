@@ -1143,9 +1143,10 @@ def _redudra_kernel_rows(z, dev):
     it; rows with an empty "like" are the siblings themselves)."""
     from ..ops import serving_kernels as sk
     from ..ops.causal_conv import conv_silu_ragged
-    from ..ops.gated_recurrence import diagonal_scan, rglru_gates
+    from ..ops.gated_recurrence import (diagonal_scan, rglru_gates,
+                                        rglru_mix)
     from ..ops.linear_recurrence import (head_norm_gate, linear_scan,
-                                         retention_prep)
+                                         retention_mix, retention_prep)
     from ..ops.norms import residual_norm
     from ..ops.rope import rope_tables
     from .state_cache import PagedStateCache
@@ -1250,10 +1251,21 @@ def _redudra_kernel_rows(z, dev):
         io = n * RH * (2 * rd + rv) * 2 + n * RH * rv * 4 \
             + 2 * NB * RH * rd * rv * 4
         fl = n * RH * 4.0 * rd * rv
-        row("linear_scan retention, %d x %d tokens" % (NB, cnt),
-            "linear_scan gla",
-            lambda: linear_scan(qq, kk, vv, dec, None, st, bt),
-            io + n * RH * 2 * rd * 2, fl)
+        if cnt > 1:
+            row("linear_scan retention (chunks), %d x %d tokens" % (NB, cnt),
+                "linear_scan gla",
+                lambda: linear_scan(qq, kk, vv, dec, None, st, bt),
+                io + n * RH * 2 * rd * 2, fl)
+        else:
+            pj = torch.randn(n, RH * (2 * rd + 2 * rv), device=dev).to(bf)
+            ro = torch.empty(n, RH * rv, device=dev, dtype=bf)
+            nq, nv = 2 * RH * rd, RH * rv
+            row("retention_step (rotary, scan, norm, gate), %d x 1 tokens"
+                % NB, "linear_scan gla",
+                lambda: retention_mix(pj[:, :nq], pj[:, nq:nq + nv],
+                                      pj[:, nq + nv:], dec, st, bt, RH, rd,
+                                      rv, rd, cos, sin, 1e-6, 0.7, ro),
+                n * RH * (2 * rd + 3 * rv) * 2 + 2 * NB * RH * rd * rv * 4)
         q16, k16 = qq.to(bf), kk.to(bf)
         dch = torch.rand(n, RH, rd, device=dev) * 0.1 + 0.9
         row("linear_scan gla (lolulorn), %d x %d tokens" % (NB, cnt), "",
@@ -1288,24 +1300,32 @@ def _redudra_kernel_rows(z, dev):
                              NB * (S + 64), dtype=bf, device=dev)
         bt = rc.begin_ragged(list(range(NB)), [cnt] * NB)
         pin = torch.randn(n, 2 * W, device=dev).to(bf)
-        row("conv (bias, no activation), " + case, "conv_silu",
-            lambda: conv_silu_ragged(pin[:, W:], cw, rc.states["conv"], bt,
-                                     zero, bf, None), n * W * 4)
-        row("conv_silu (savovik), " + case, "",
-            lambda: conv_silu_ragged(pin[:, W:], cw, rc.states["conv"], bt,
-                                     zero, bf), n * W * 4)
         u = torch.randn(n, W, device=dev).to(bf)
-        row("rglru_gates (both block products, gates), " + case,
-            "sigmoid_pow",
-            lambda: rglru_gates(u, wr, zero, wi, zero, zero),
-            n * W * 10 + 4 * W * (W // nbk), 4.0 * n * W * (W // nbk))
-        row("sigmoid_pow (lolulorn: bf16 in, fp32 out), " + case, "",
-            lambda: sk.sigmoid_pow(u, zero, 1.0 / 16), n * W * 6)
-        a, bb = rglru_gates(u, wr, zero, wi, zero, zero)
-        row("diagonal_scan (gated read-out), " + case, "selective_scan",
-            lambda: diagonal_scan(a, bb, rc.states["rec"], bt, pin[:, :W],
-                                  "gelu_tanh", bf),
-            n * W * 12 + 2 * NB * W * 4)
+        a = torch.randn(n, W, device=dev)
+        if cnt > 1:
+            row("conv (bias, no activation), " + case, "conv_silu",
+                lambda: conv_silu_ragged(pin[:, W:], cw, rc.states["conv"],
+                                         bt, zero, bf, None), n * W * 4)
+            row("conv_silu (savovik), " + case, "",
+                lambda: conv_silu_ragged(pin[:, W:], cw, rc.states["conv"],
+                                         bt, zero, bf), n * W * 4)
+            row("rglru_gates (both block products, gates), " + case,
+                "sigmoid_pow",
+                lambda: rglru_gates(u, wr, zero, wi, zero, zero),
+                n * W * 10 + 4 * W * (W // nbk), 4.0 * n * W * (W // nbk))
+            row("sigmoid_pow (lolulorn: bf16 in, fp32 out), " + case, "",
+                lambda: sk.sigmoid_pow(u, zero, 1.0 / 16), n * W * 6)
+            a, bb = rglru_gates(u, wr, zero, wi, zero, zero)
+            row("diagonal_scan (gated read-out), " + case, "selective_scan",
+                lambda: diagonal_scan(a, bb, rc.states["rec"], bt,
+                                      pin[:, :W], "gelu_tanh", bf),
+                n * W * 12 + 2 * NB * W * 4)
+        else:
+            row("rglru_step (conv, gates, scan, read-out), " + case,
+                "selective_scan",
+                lambda: rglru_mix(pin, cw, zero, rc.states["conv"], wr, zero,
+                                  wi, zero, zero, rc.states["rec"], bt),
+                n * W * 26 + 4 * W * (W // nbk))
         bc = (torch.randn(n, 2 * SN, device=dev) * 0.1).to(bf)
         so = torch.empty(n, W, device=dev, dtype=bf)
         row("selective_scan (savovik), " + case, "",
@@ -1314,7 +1334,7 @@ def _redudra_kernel_rows(z, dev):
                                       rc.states["sel"], bt, 1.0, so),
             n * W * 10 + n * 2 * SN * 2 + 2 * NB * W * SN * 4)
         rc.end_step()
-        del rc, pin, u, a, bb
+        del rc, pin, u, a
     gu = torch.randn(T, 2 * F, device=dev).to(bf)
     row("glu silu (also lolulorn's)", "", lambda: sk.glu(gu, 0), T * F * 6)
     lg = torch.randn(64, 32000, device=dev).to(bf)

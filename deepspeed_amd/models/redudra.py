@@ -38,10 +38,8 @@ import torch.nn.functional as F
 
 from ..inference.state_cache import PagedStateCache
 from ..ops.activations import softcap_rows
-from ..ops.causal_conv import conv_silu_ragged
-from ..ops.gated_recurrence import diagonal_scan, rglru_gates
-from ..ops.linear_recurrence import (head_norm_gate, linear_scan,
-                                     retention_prep)
+from ..ops.gated_recurrence import rglru_mix
+from ..ops.linear_recurrence import retention_mix
 from ..ops.norms import embed_rows, residual_norm
 from .lolulorn import GatedMLP, PostNorm
 from .savovik import GroupedAttention, rot_tables
@@ -144,14 +142,9 @@ class RGLRUMixer(nn.Module):
 
     def forward(self, h, cache: PagedStateCache, stream, states):
         b = cache.batch
-        C = self.inner
-        proj = F.linear(h, self.w_in, self.b_in)
-        u = conv_silu_ragged(proj[:, C:], self.conv, states["conv"], b,
-                             self.conv_b, h.dtype, act=None)
-        a, z = rglru_gates(u, self.w_r, self.b_r, self.w_i, self.b_i,
-                           self.lam)
-        y = diagonal_scan(a, z, states["rec"], b, proj[:, :C], "gelu_tanh",
-                          h.dtype)
+        y = rglru_mix(F.linear(h, self.w_in, self.b_in), self.conv,
+                      self.conv_b, states["conv"], self.w_r, self.b_r,
+                      self.w_i, self.b_i, self.lam, states["rec"], b)
         return F.linear(y, self.w_o)
 
 
@@ -195,20 +188,19 @@ class WindowRetentionMixer(nn.Module):
 
     def forward(self, h, cache: PagedStateCache, stream, states):
         b = cache.batch
-        T, H = h.shape[0], self.heads
         n0, n_l, nq, nv = self.att.n_in, self.att.n_out, self.n_qk, self.n_v
         proj = F.linear(h, self.w_in)
-        both = torch.empty(T, n_l + nv, dtype=h.dtype, device=h.device)
+        both = torch.empty(h.shape[0], n_l + nv, dtype=h.dtype, device=h.device)
         self.att.run(proj[:, :n0], cache, stream, out=both[:, :n_l],
                      out_scale=self.left_scale)
         cos, sin = rot_tables(self.rot, cache.max_seq, h.device) \
             if self.rot_dims else (None, None)
-        q, k = retention_prep(proj[:, n0:n0 + 2 * nq], b, H, self.dim,
-                              self.rot_dims, cos, sin, self.dim ** -0.5)
-        v = proj[:, n0 + 2 * nq:n0 + 2 * nq + nv].view(T, H, self.vdim)
-        o = linear_scan(q, k, v, self.head_decay, None, states["rec"], b)
-        head_norm_gate(o, None, proj[:, n0 + 2 * nq + nv:], self.eps,
-                       h.dtype, out_scale=self.right_scale, out=both[:, n_l:])
+        retention_mix(proj[:, n0:n0 + 2 * nq],
+                      proj[:, n0 + 2 * nq:n0 + 2 * nq + nv],
+                      proj[:, n0 + 2 * nq + nv:], self.head_decay,
+                      states["rec"], b, self.heads, self.dim, self.vdim,
+                      self.rot_dims, cos, sin, self.eps, self.right_scale,
+                      both[:, n_l:])
         return F.linear(both, self.w_o)
 
 

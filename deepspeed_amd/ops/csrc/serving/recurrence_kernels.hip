@@ -305,6 +305,168 @@ __global__ __launch_bounds__(NT) void diagonal_scan_short_k(
   *Sg = S;
 }
 
+// One token per sequence, 16-bit: convolution, tail shift, both gate products,
+// gates, state update and gated read-out of one block of channels of up to 16
+// sequences in one workgroup (it owns the block's channels: nobody else reads
+// or shifts their tails). proj row = [ y (W) | x (W) ].
+constexpr int RS_W = 8;  // waves
+
+__global__ __launch_bounds__(64 * RS_W) void rglru_step_k(
+    const bf16* __restrict__ proj, int ld_proj, const bf16* __restrict__ cw,
+    const float* __restrict__ cb, bf16* __restrict__ tail, int64_t tail_stride, int taps,
+    const bf16* __restrict__ wr, const bf16* __restrict__ wi, const float* __restrict__ br,
+    const float* __restrict__ bi, const float* __restrict__ lam, float* __restrict__ state,
+    const int* __restrict__ seq_slot, const int* __restrict__ seq_start, bf16* __restrict__ out,
+    int nseq, int n, int W, float c) {
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  bf16* sU = reinterpret_cast<bf16*>(smem);  // [16][pitch]
+  const int pitch = (n + 31) / 32 * 32 + 8;
+  const int t0 = blockIdx.x * 16, blk = blockIdx.y;
+  const int kept = taps - 1;
+  for (int i = threadIdx.x; i < 16 * pitch; i += 64 * RS_W) {
+    const int tk = i / pitch, k = i - tk * pitch;
+    const int t = t0 + tk;
+    float u = 0.f;
+    if (k < n && t < nseq) {
+      const int ch = blk * n + k;
+      const bf16 xin = proj[(int64_t)t * ld_proj + W + ch];
+      const int pos = seq_start[t];
+      bf16* tl = tail + (int64_t)seq_slot[t] * tail_stride + ch;
+      const bf16* w = cw + (int64_t)ch * taps;
+      u = ld(w + kept) * ld(&xin);
+      for (int j = 1; j <= kept; ++j)
+        if (pos - j >= 0) u += ld(w + kept - j) * ld(tl + (int64_t)(kept - j) * W);
+      u += cb[ch];
+      for (int j = 0; j + 1 < kept; ++j) tl[(int64_t)j * W] = tl[(int64_t)(j + 1) * W];
+      if (kept > 0) tl[(int64_t)(kept - 1) * W] = xin;
+    }
+    st(sU + i, u);
+  }
+  __syncthreads();
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int l15 = lane & 15, quad = lane >> 4;
+  const bool vec = (n & 7) == 0;
+  for (int ot = wave; ot * 16 < n; ot += RS_W) {
+    const int o = ot * 16 + l15;
+    const short* rr = reinterpret_cast<const short*>(wr) + ((int64_t)blk * n + o) * n;
+    const short* ri = reinterpret_cast<const short*>(wi) + ((int64_t)blk * n + o) * n;
+    auto get = [&](const short* row, int k) {
+      short8 x = {0, 0, 0, 0, 0, 0, 0, 0};
+      if (o < n) {
+        if (vec) {
+          if (k < n) x = *reinterpret_cast<const short8*>(row + k);
+        } else {
+#pragma unroll
+          for (int e = 0; e < 8; ++e)
+            if (k + e < n) x[e] = row[k + e];
+        }
+      }
+      return x;
+    };
+    typedef __attribute__((ext_vector_type(8))) __bf16 frag;
+    floatx4 ar = {0.f, 0.f, 0.f, 0.f}, ai = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+    for (int kk = 0; kk < n; kk += 32) {
+      const int k = kk + quad * 8;
+      const frag fa = *reinterpret_cast<const frag*>(sU + l15 * pitch + k);
+      ar = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fa, __builtin_bit_cast(frag, get(rr, k)), ar, 0,
+                                                   0, 0);
+      ai = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fa, __builtin_bit_cast(frag, get(ri, k)), ai, 0,
+                                                   0, 0);
+    }
+    if (o >= n) continue;
+    const int ch = blk * n + o;
+    const float rate = c * softplus_(lam[ch]), cr = br[ch], ci = bi[ch];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int t = t0 + quad * 4 + e;
+      if (t < nseq) {
+        float a, b;
+        rglru_pair<false>(ar[e] + cr, ai[e] + ci, ld(sU + (quad * 4 + e) * pitch + o), rate, a, b);
+        float* Sg = state + (int64_t)seq_slot[t] * W + ch;
+        const float S = a * *Sg + b;
+        *Sg = S;
+        st(out + (int64_t)t * W + ch,
+           S * gate_act<false>(ld(proj + (int64_t)t * ld_proj + ch), 0));
+      }
+    }
+  }
+}
+
+// ------------------------------ retention, one token per sequence, in one pass
+// A workgroup owns one head of one sequence: rotation of q and k (HALF
+// pairing, keys then times k_scale), S <- g S + k v^T, o = S^T q, RMS norm of
+// o over the head, times SiLU(gate) and out_scale. CW neighbouring threads
+// hold neighbouring columns; RT_T / CW groups share the rows.
+constexpr int RT_T = 1024;
+
+template <typename T, int CW>
+__global__ __launch_bounds__(RT_T) void retention_step_k(
+    const T* __restrict__ qk, int ld_qk, const T* __restrict__ v, int ld_v,
+    const T* __restrict__ gate, int ld_gate, const float* __restrict__ cosT,
+    const float* __restrict__ sinT, const int* __restrict__ tok_pos,
+    const float* __restrict__ decay, float* __restrict__ state, const int* __restrict__ seq_slot,
+    T* __restrict__ out, int ld_out, int H, int dim, int vdim, int rot_dims, float k_scale,
+    float eps, float out_scale) {
+  constexpr bool EXACT = sizeof(T) == 4;
+  constexpr int RG = RT_T / CW;
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  float* sq = reinterpret_cast<float*>(smem);  // [dim]
+  float* sk = sq + dim;                        // [dim]
+  float* so = sk + dim;                        // [vdim]
+  float* sp = so + vdim;                       // [RT_T]
+  const int t = blockIdx.x, h = blockIdx.y;
+  const int half = rot_dims >> 1;
+  const float* cs = cosT + (int64_t)tok_pos[t] * half;
+  const float* sn = sinT + (int64_t)tok_pos[t] * half;
+  for (int i = threadIdx.x; i < 2 * dim; i += RT_T) {
+    const bool is_k = i >= dim;
+    const int c = is_k ? i - dim : i;
+    const T* hd = qk + (int64_t)t * ld_qk + (is_k ? (H + h) * dim : h * dim);
+    float x = ld(hd + c);
+    if (c < rot_dims) {
+      const bool second = c >= half;
+      const int f = second ? c - half : c;
+      const float y = ld(hd + (second ? f : c + half));
+      x = second ? x * cs[f] + y * sn[f] : x * cs[f] - y * sn[f];
+    }
+    sq[i] = is_k ? x * k_scale : x;
+  }
+  __syncthreads();
+  const float g = decay[h];
+  float* Sh = state + ((int64_t)seq_slot[t] * H + h) * dim * (int64_t)vdim;
+  const int cl = threadIdx.x % CW, rg = threadIdx.x / CW;
+  for (int c0 = 0; c0 < vdim; c0 += CW) {
+    const int c = c0 + cl;
+    float acc = 0.f;
+    if (c < vdim) {
+      const float vc = ld(v + (int64_t)t * ld_v + h * vdim + c);
+#pragma unroll 8
+      for (int d = rg; d < dim; d += RG) {
+        float* p = Sh + (int64_t)d * vdim + c;
+        const float S = g * *p + sk[d] * vc;
+        *p = S;
+        acc += sq[d] * S;
+      }
+    }
+    sp[threadIdx.x] = acc;
+    __syncthreads();
+    if (rg == 0 && c < vdim) {
+      float o = 0.f;
+      for (int r = 0; r < RG; ++r) o += sp[r * CW + cl];
+      so[c] = o;
+    }
+    __syncthreads();
+  }
+  float ss = 0.f;
+  for (int c = threadIdx.x; c < vdim; c += RT_T) ss += so[c] * so[c];
+  const float inv = rsqrtf(block_sum(ss, sp) / (float)vdim + eps) * out_scale;
+  for (int c = threadIdx.x; c < vdim; c += RT_T) {
+    const float z = ld(gate + (int64_t)t * ld_gate + h * vdim + c);
+    st(out + (int64_t)t * ld_out + h * vdim + c, so[c] * inv * gate_act<EXACT>(z, 1));
+  }
+}
+
 // ------------------------- matrix-state recurrence with a fixed decay, chunks
 // S <- g S + k v^T, o = S^T q per head, RC tokens at a time on matrix cores:
 // with a chunk's tokens 0..n-1 and the state S0 before it,
@@ -718,6 +880,48 @@ int dsv_retention_chunk(const float* q, const float* k, const void* v, int ld_v,
                                       dim, vdim, q_scale, s);
   return launch_retention_chunk<128>(q, k, v, ld_v, decay, state, cu, seq_slot, out, nseq, G, H,
                                      dim, vdim, q_scale, s);
+}
+
+// one token per sequence: flat token i is sequence i's
+int dsv_rglru_step(const void* proj, int ld_proj, const void* cw, const float* cb, void* tail,
+                   int64_t tail_stride, int taps, const void* wr, const void* wi, const float* br,
+                   const float* bi, const float* lam, float* state, const int* seq_slot,
+                   const int* seq_start, void* out, int nseq, int blocks, int n, float c,
+                   hipStream_t s) {
+  if (nseq <= 0) return 0;
+  if (blocks < 1 || blocks > 65535 || n < 1 || taps < 1 || ld_proj < 2 * blocks * n) return -1;
+  if ((uintptr_t)wr % 16 || (uintptr_t)wi % 16) return -2;
+  const size_t lds = (size_t)16 * ((n + 31) / 32 * 32 + 8) * 2;
+  if (lds > 48 * 1024) return -3;
+  rglru_step_k<<<dim3((nseq + 15) / 16, blocks), 64 * RS_W, lds, s>>>(
+      (const bf16*)proj, ld_proj, (const bf16*)cw, cb, (bf16*)tail, tail_stride, taps,
+      (const bf16*)wr, (const bf16*)wi, br, bi, lam, state, seq_slot, seq_start, (bf16*)out, nseq,
+      n, blocks * n, c);
+  return (int)hipGetLastError();
+}
+
+// one token per sequence; qk row = [ q (H x dim) | k (H x dim) ]
+int dsv_retention_step(const void* qk, int ld_qk, const void* v, int ld_v, const void* gate,
+                       int ld_gate, const float* cosT, const float* sinT, const int* tok_pos,
+                       const float* decay, float* state, const int* seq_slot, void* out,
+                       int ld_out, int dt, int nseq, int H, int dim, int vdim, int rot_dims,
+                       float k_scale, float eps, float out_scale, hipStream_t s) {
+  if (nseq <= 0) return 0;
+  if (H < 1 || H > 65535 || dim < 1 || vdim < 1) return -1;
+  if (rot_dims < 0 || (rot_dims & 1) || rot_dims > dim) return -2;
+  if (rot_dims > 0 && (!cosT || !sinT)) return -2;
+  const size_t lds = ((size_t)2 * dim + vdim + RT_T) * 4;
+  if (lds > 48 * 1024) return -3;
+#define RSTEP(CW)                                                                               \
+  BY_DTYPE(dt, (retention_step_k<T, CW><<<dim3(nseq, H), RT_T, lds, s>>>(                        \
+                   (const T*)qk, ld_qk, (const T*)v, ld_v, (const T*)gate, ld_gate, cosT, sinT,  \
+                   tok_pos, decay, state, seq_slot, (T*)out, ld_out, H, dim, vdim, rot_dims,     \
+                   k_scale, eps, out_scale)))
+  if (vdim <= 64) RSTEP(64);
+  else if (vdim <= 128) RSTEP(128);
+  else RSTEP(256);
+#undef RSTEP
+  return (int)hipGetLastError();
 }
 
 }  // extern "C"

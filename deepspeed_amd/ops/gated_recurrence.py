@@ -13,6 +13,9 @@ ragged batches.
   ``1 - a^2`` is evaluated as ``-expm1(2 log a)`` (exact where a is near 1).
 * ``diagonal_scan``: ``S <- a * S + b`` per channel from the slot's state (zero
   at a sequence's start), read out as ``S * act(gate)``.
+* ``rglru_mix``: the recurrent block between its input and output projections
+  (short convolution, gates, scan, gated read-out); one kernel where every
+  sequence brings a single token.
 
 Everything is fp32 whatever the storage type of u, the matrices and the gate
 rows (products of 16-bit operands accumulate in fp32 and stay fp32).
@@ -20,6 +23,8 @@ rows (products of 16-bit operands accumulate in fp32 and stay fp32).
 
 import torch
 import torch.nn.functional as F
+
+from .causal_conv import conv_silu_ragged
 
 RGLRU_C = 8.0
 
@@ -76,3 +81,20 @@ def diagonal_scan(a, b, state, batch, gate=None, act="gelu_tanh",
         out = out * (F.gelu(g, approximate="tanh") if act == "gelu_tanh"
                      else F.silu(g))
     return out.to(out_dtype)
+
+
+def rglru_mix(proj, conv_w, conv_b, conv_state, w_r, b_r, w_i, b_i, lam,
+              state, batch, c=RGLRU_C):
+    """proj [T, 2W] = y | x: ``scan(gates(conv(x))) * gelu_tanh(y)`` as [T, W]
+    in proj's dtype. conv_state [slots, taps-1, W] and state [slots, W] (fp32)
+    are advanced in place."""
+    W = proj.shape[1] // 2
+    if proj.is_cuda and _sk().enabled() and \
+            _sk().rglru_step_ok(proj, batch, w_r.shape[1]):
+        return _sk().rglru_step(proj, conv_w, conv_b, conv_state, w_r, b_r,
+                                w_i, b_i, lam, state, batch, c)
+    u = conv_silu_ragged(proj[:, W:], conv_w, conv_state, batch, conv_b,
+                         proj.dtype, act=None)
+    a, b = rglru_gates(u, w_r, b_r, w_i, b_i, lam, c)
+    return diagonal_scan(a, b, state, batch, proj[:, :W], "gelu_tanh",
+                         proj.dtype)

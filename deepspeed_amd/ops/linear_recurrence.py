@@ -35,6 +35,9 @@ Around the scan:
   by the heads (or none), times ``silu(gate)`` or ``sigmoid(gate)``.
 * ``retention_prep``: queries and keys of a retention layer (the plain form
   with one fixed decay per head): partial rotary positions, keys scaled.
+* ``retention_mix``: a retention layer between its input and output
+  projections (prologue, recurrence, normed and gated read-out); one kernel
+  where every sequence brings a single token.
 """
 
 import torch
@@ -239,3 +242,26 @@ def retention_prep(proj, batch, heads, dim, rot_dims, cos, sin, k_scale,
         rotate(q, batch.tok_pos, cos, sin, rot_dims)
         rotate(k, batch.tok_pos, cos, sin, rot_dims)
     return q, k * k_scale
+
+
+def retention_mix(qk, v, gate, decay, state, batch, heads, dim, vdim,
+                  rot_dims, cos, sin, eps, out_scale=1.0, out=None):
+    """qk [T, 2*heads*dim] = q | k, v and gate [T, heads*vdim] (column slices
+    are fine); decay [heads] fp32; state [slots, heads, dim, vdim] fp32,
+    advanced in place. Rotate-half positions on q and k, keys then times
+    ``dim ** -0.5``; ``S <- decay S + k v^T``, ``o = S^T q``; every head's o
+    divided by its root mean square, times ``silu(gate) * out_scale``.
+    Returns [T, heads*vdim] in qk's dtype, written into ``out`` when given."""
+    T = qk.shape[0]
+    if out is None:
+        out = torch.empty(T, heads * vdim, dtype=qk.dtype, device=qk.device)
+    if qk.is_cuda and _sk().enabled() and \
+            _sk().retention_step_ok(batch, dim, vdim):
+        return _sk().retention_step(qk, v, gate, decay, state, batch, heads,
+                                    dim, vdim, rot_dims, cos, sin,
+                                    dim ** -0.5, eps, out_scale, out)
+    q, k = retention_prep(qk, batch, heads, dim, rot_dims, cos, sin,
+                          dim ** -0.5)
+    o = linear_scan(q, k, v.view(T, heads, vdim), decay, None, state, batch)
+    return head_norm_gate(o, None, gate, eps, qk.dtype, "silu", out_scale,
+                          out)

@@ -1071,5 +1071,76 @@ def diagonal_scan(a, b, state, batch, gate, act, out_dtype):
     return out
 
 
+def single_tokens(batch):
+    """Every sequence of the step brings exactly one token."""
+    return batch.n_tokens == batch.n_seqs and max(batch.counts) == 1
+
+
+STEP_MAX = 256      # more requests at once: the kernels that tile tokens
+
+
+def rglru_step_ok(proj, batch, n):
+    return proj.dtype == torch.bfloat16 and single_tokens(batch) and \
+        batch.n_seqs <= STEP_MAX and 16 * ((n + 31) // 32 * 32 + 8) * 2 <= 48 * 1024
+
+
+def rglru_step(proj, conv_w, conv_b, conv_state, w_r, b_r, w_i, b_i, lam,
+               state, batch, c):
+    T = proj.shape[0]
+    blocks, n, _ = w_r.shape
+    W, taps = blocks * n, conv_w.shape[1]
+    _rows_ok(proj)
+    assert T == batch.n_tokens and proj.shape[1] == 2 * W
+    assert proj.dtype == conv_w.dtype == conv_state.dtype == torch.bfloat16
+    assert w_r.dtype == w_i.dtype == torch.bfloat16
+    assert w_i.shape == w_r.shape == (blocks, n, n)
+    assert conv_w.shape == (W, taps) and conv_w.is_contiguous()
+    assert conv_state.shape[1:] == (taps - 1, W)
+    assert conv_state.stride(2) == 1 and (taps == 1
+                                          or conv_state.stride(1) == W)
+    assert conv_b.numel() == b_r.numel() == b_i.numel() == lam.numel() == W
+    assert state.dtype == torch.float32 and state.is_contiguous()
+    assert state.shape[1:] == (W,)
+    out = torch.empty(T, W, dtype=proj.dtype, device=proj.device)
+    _check(load("recur").dsv_rglru_step(
+        _vp(proj), _i(proj.stride(0)), _p(conv_w),
+        _p(_f32(conv_b).contiguous()), _vp(conv_state),
+        _l(conv_state.stride(0)), _i(taps), _p(w_r), _p(w_i),
+        _p(_f32(b_r).contiguous()), _p(_f32(b_i).contiguous()),
+        _p(_f32(lam).contiguous()), _p(state), _p(batch.seq_slot),
+        _p(batch.seq_start), _p(out), _i(batch.n_seqs), _i(blocks), _i(n),
+        _f(c), _stream()), "rglru_step")
+    return out
+
+
+def retention_step_ok(batch, dim, vdim):
+    return single_tokens(batch) and (2 * dim + vdim + 1024) * 4 <= 48 * 1024
+
+
+def retention_step(qk, v, gate, decay, state, batch, heads, dim, vdim,
+                   rot_dims, cos, sin, k_scale, eps, out_scale, out):
+    T = qk.shape[0]
+    for t in (qk, v, gate, out):
+        _rows_ok(t)
+        assert t.dtype == qk.dtype and t.shape[0] == T
+    assert T == batch.n_tokens and qk.shape[1] == 2 * heads * dim
+    assert v.shape[1] == gate.shape[1] == out.shape[1] == heads * vdim
+    assert decay.dtype == torch.float32 and decay.shape == (heads,)
+    assert state.dtype == torch.float32 and state.is_contiguous()
+    assert state.shape[1:] == (heads, dim, vdim)
+    if rot_dims:
+        assert cos.shape[1] == rot_dims // 2 and cos.shape[0] >= batch.max_ctx
+        assert cos.dtype == torch.float32 and sin.shape == cos.shape
+    _check(load("recur").dsv_retention_step(
+        _vp(qk), _i(qk.stride(0)), _vp(v), _i(v.stride(0)), _vp(gate),
+        _i(gate.stride(0)), _p(cos if rot_dims else None),
+        _p(sin if rot_dims else None), _p(batch.tok_pos),
+        _p(decay.contiguous()), _p(state), _p(batch.seq_slot), _vp(out),
+        _i(out.stride(0)), _i(_dt(qk)), _i(batch.n_seqs), _i(heads), _i(dim),
+        _i(vdim), _i(rot_dims), _f(k_scale), _f(eps), _f(out_scale),
+        _stream()), "retention_step")
+    return out
+
+
 if __name__ == "__main__":
     print(build(force="--if-stale" not in sys.argv))

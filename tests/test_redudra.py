@@ -1130,6 +1130,85 @@ def test_scan_with_a_fixed_decay_against_eager(H, d, dv, vdt, monkeypatch):
 
 
 @pytest.mark.gpu
+@pytest.mark.parametrize("blocks,n,taps,N", [
+    (3, 5, 4, 3), (2, 72, 4, 1), (1, 20, 1, 5), (4, 64, 2, 17), (2, 256, 4, 40),
+    (1, 200, 7, 2)])
+def test_single_token_recurrence_step_against_its_parts(blocks, n, taps, N,
+                                                        monkeypatch):
+    """One fused kernel against convolution, gates and scan one by one, over
+    several steps, from the first token on; slots in no order."""
+    from deepspeed_amd.ops import serving_kernels as sk
+    from deepspeed_amd.ops.gated_recurrence import rglru_mix
+    W, bf = blocks * n, torch.bfloat16
+    wr, wi = ((rnd(blocks, n, n, seed=k) * n ** -0.5).to(DEV, bf)
+              for k in (1, 2))
+    br, bi, lam, cb = (rnd(W, seed=k).to(DEV) for k in (3, 4, 5, 6))
+    cw = rnd(W, taps, seed=7).to(DEV, bf)
+    slots = torch.randperm(N + 2, generator=torch.Generator()
+                           .manual_seed(N)).tolist()[:N]
+
+    def run(fused):
+        cache = PagedStateCache([], {"conv": ((taps - 1, W), bf),
+                                     "rec": ((W,), torch.float32)}, N + 2,
+                                64 * N, block_size=8, device=DEV, dtype=bf)
+        for s in slots[1::2]:            # half of them go on from somewhere
+            cache.states["conv"][s] = rnd(taps - 1, W, seed=s).to(DEV, bf)
+            cache.states["rec"][s] = rnd(W, seed=50 + s).to(DEV)
+            cache.lens[s] = 9
+        outs = []
+        for k in range(taps + 2):
+            bt = cache.begin_ragged(slots, [1] * N)
+            proj = rnd(N, 2 * W + 8, seed=90 + k).to(DEV, bf)[:, 8:]
+            args = (proj, cw, cb, cache.states["conv"], wr, br, wi, bi, lam,
+                    cache.states["rec"], bt)
+            if fused:
+                assert sk.rglru_step_ok(proj, bt, n)
+            outs.append(rglru_mix(*args))
+            cache.end_step()
+        return torch.stack(outs), cache.states["conv"], cache.states["rec"]
+
+    got = run(True)
+    monkeypatch.setattr(sk, "STEP_MAX", 0)
+    want = run(False)
+    monkeypatch.setenv("DS_AMD_SERVING_EAGER", "1")
+    eager = run(False)
+    for ref in (want, eager):
+        near(got[0], ref[0], bf)
+        assert torch.equal(got[1], ref[1])
+        # a convolution's sum can round to the neighbouring 16-bit value
+        near(got[2], ref[2], bf)
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("H,d,dv,dims,N", [
+    (3, 8, 5, 6, 2), (2, 64, 64, 64, 1), (2, 128, 256, 32, 9),
+    (1, 36, 300, 0, 3), (4, 16, 128, 16, 33)])
+def test_single_token_retention_step_against_its_parts(H, d, dv, dims, N,
+                                                       dtype, monkeypatch):
+    from deepspeed_amd.ops.linear_recurrence import retention_mix
+    from deepspeed_amd.ops.rope import rope_tables
+    cos, sin = rope_tables(dims, 2048, 500.0, device=DEV) if dims \
+        else (None, None)
+    dec = torch.tensor([0.99, 1.0, 0.0, 0.3][:H]).to(DEV)
+    x = rnd(N, 8 + 2 * H * (d + dv)).to(DEV, dtype)
+    st0 = rnd(N, H, d, dv, seed=3).to(DEV)
+    nq, nv = 8 + 2 * H * d, H * dv
+
+    def run():
+        _, bt = begun({}, [7 * i for i in range(N)], [1] * N)
+        st, wide = st0.clone(), torch.zeros(N, nv + 8, device=DEV,
+                                            dtype=dtype)
+        retention_mix(x[:, 8:nq], x[:, nq:nq + nv], x[:, nq + nv:], dec, st,
+                      bt, H, d, dv, dims, cos, sin, 1e-5, 0.7, wide[:, 8:])
+        return wide, st
+
+    got, want = _both(monkeypatch, run)
+    near(got[0], want[0], dtype)
+    near(got[1], want[1], torch.float32)
+
+
+@pytest.mark.gpu
 @pytest.mark.parametrize("counts", [[1, 70, 20], [64, 63, 65], [2, 200, 128],
                                     [16]])
 @pytest.mark.parametrize("H,G,d,dv", [(3, 3, 8, 4), (2, 2, 64, 64),

@@ -31,27 +31,26 @@ __device__ __forceinline__ float sigmoid_(float x) {
 __device__ __forceinline__ float softplus_(float x) {
   return x > 20.f ? x : log1pf(expf(x));
 }
-// 1 - exp(y) for y <= 0: the series where the difference would cancel
-template <bool EXACT>
-__device__ __forceinline__ float one_minus_exp(float y) {
-  if (EXACT) return -expm1f(y);
-  const float series =
-      -y * (1.f + y * (1.f / 2) *
-                      (1.f + y * (1.f / 3) *
-                                 (1.f + y * (1.f / 4) *
-                                            (1.f + y * (1.f / 5) *
-                                                       (1.f + y * (1.f / 6) *
-                                                                  (1.f + y * (1.f / 7)))))));
-  return y > -0.4f ? series : 1.f - exp_<false>(y);
-}
-
-// (r, i pre-activations with bias) -> a and b of S <- a S + b
+// (r, i pre-activations with bias) -> a and b of S <- a S + b. 1 - a^2 is
+// 1 - exp(y) with y = 2 log a <= 0; where that would cancel, the series.
 template <bool EXACT>
 __device__ __forceinline__ void rglru_pair(float zr, float zi, float u, float rate, float& a,
                                            float& b) {
   const float la = -sigmoid_<EXACT>(zr) * rate;  // rate = c * softplus(lam)
   a = exp_<EXACT>(la);
-  b = sqrtf(one_minus_exp<EXACT>(2.f * la)) * (sigmoid_<EXACT>(zi) * u);
+  const float y = 2.f * la;
+  float m;
+  if (EXACT) {
+    m = -expm1f(y);
+  } else {
+    const float series =
+        -y * (1.f + y * (1.f / 2) *
+                        (1.f + y * (1.f / 3) *
+                                   (1.f + y * (1.f / 4) *
+                                              (1.f + y * (1.f / 5) * (1.f + y * (1.f / 6))))));
+    m = y > -0.25f ? series : 1.f - a * a;
+  }
+  b = (EXACT ? sqrtf(m) : __builtin_amdgcn_sqrtf(m)) * (sigmoid_<EXACT>(zi) * u);
 }
 
 // Gates from finished products: zr, zi [blocks, T, n] float (no bias yet).
@@ -89,10 +88,12 @@ __global__ __launch_bounds__(NT) void rglru_gates_mfma_k(
     const bf16* __restrict__ u, const bf16* __restrict__ wr, const bf16* __restrict__ wi,
     const float* __restrict__ br, const float* __restrict__ bi, const float* __restrict__ lam,
     float* __restrict__ a, float* __restrict__ b, int Ttok, int n, int W, float c) {
-  constexpr int TM = 16 * WM, TN = 16 * WN * NN;
-  __shared__ __attribute__((aligned(16))) short sU[TM * GKP];
-  __shared__ __attribute__((aligned(16))) short sR[TN * GKP];
-  __shared__ __attribute__((aligned(16))) short sI[TN * GKP];
+  constexpr int TM = 16 * WM, TN = 16 * WN * NN, ZP = TN + 4;
+  constexpr int LDS_IN = (TM + 2 * TN) * GKP * 2, LDS_OUT = 2 * TM * ZP * 4;
+  __shared__ __attribute__((aligned(16))) char smem[LDS_IN > LDS_OUT ? LDS_IN : LDS_OUT];
+  short* sU = reinterpret_cast<short*>(smem);  // [TM][GKP]
+  short* sR = sU + TM * GKP;                   // [TN][GKP]
+  short* sI = sR + TN * GKP;                   // [TN][GKP]
   const int t0 = blockIdx.x * TM, blk = blockIdx.y, o0 = blockIdx.z * TN;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int wm = wave % WM, wn = wave / WM;
@@ -180,6 +181,51 @@ __global__ __launch_bounds__(NT) void rglru_gates_mfma_k(
       }
     }
     __syncthreads();
+  }
+  if (TN == 64 && (n & 3) == 0) {
+    // the products go through LDS once more, so that a thread finishes four
+    // neighbouring channels and whole 16-byte groups are stored
+    float* zr = reinterpret_cast<float*>(smem);  // [TM][ZP]
+    float* zi = zr + TM * ZP;
+#pragma unroll
+    for (int j = 0; j < NN; ++j)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const int at = (wm * 16 + quad * 4 + e) * ZP + (wn * NN + j) * 16 + l15;
+        zr[at] = ar[j][e];
+        zi[at] = ai[j][e];
+      }
+    __syncthreads();
+    const int o4 = (threadIdx.x & 15) * 4;
+    if (o0 + o4 >= n) return;
+    const int ch = blk * n + o0 + o4;
+    float rate[4], cr[4], ci[4];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      rate[e] = c * softplus_(lam[ch + e]);
+      cr[e] = br[ch + e];
+      ci[e] = bi[ch + e];
+    }
+#pragma unroll
+    for (int r = threadIdx.x >> 4; r < TM; r += NT / 16) {
+      const int64_t t = t0 + r;
+      if (t >= Ttok) break;
+      const float4 xr = *reinterpret_cast<const float4*>(zr + r * ZP + o4);
+      const float4 xi = *reinterpret_cast<const float4*>(zi + r * ZP + o4);
+      const uint2 xu = *reinterpret_cast<const uint2*>(u + t * W + ch);
+      float4 av, bv;
+      rglru_pair<false>(xr.x + cr[0], xi.x + ci[0], __uint_as_float(xu.x << 16), rate[0], av.x,
+                        bv.x);
+      rglru_pair<false>(xr.y + cr[1], xi.y + ci[1], __uint_as_float(xu.x & 0xffff0000u), rate[1],
+                        av.y, bv.y);
+      rglru_pair<false>(xr.z + cr[2], xi.z + ci[2], __uint_as_float(xu.y << 16), rate[2], av.z,
+                        bv.z);
+      rglru_pair<false>(xr.w + cr[3], xi.w + ci[3], __uint_as_float(xu.y & 0xffff0000u), rate[3],
+                        av.w, bv.w);
+      *reinterpret_cast<float4*>(a + t * W + ch) = av;
+      *reinterpret_cast<float4*>(b + t * W + ch) = bv;
+    }
+    return;
   }
 #pragma unroll
   for (int j = 0; j < NN; ++j) {
@@ -672,42 +718,53 @@ __global__ __launch_bounds__(256) void retention_chunk_k(
     if (base + RC < cnt) fetch(base + RC);
 
     // masked, decayed scores: p[jt][j] for key 16 jt + 4 quad + j, token l15
+    // (tiles above the diagonal are made and masked too: four independent
+    // chains of products fill the pipe better than a wave-dependent number)
     floatx4 p[4];
 #pragma unroll
-    for (int jt = 0; jt < 4; ++jt) {
-      floatx4 acc = {0.f, 0.f, 0.f, 0.f};
-      if (jt <= w) {
+    for (int jt = 0; jt < 4; ++jt) p[jt] = (floatx4){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int ks = 0; ks < KS; ++ks) {
-          const int at = swz(jt * 16 + l15, ks * 32 + quad * 8, DP);
-          const bf16x8 kh = *reinterpret_cast<const bf16x8*>(Kh + at);
-          const bf16x8 kl = *reinterpret_cast<const bf16x8*>(Kl + at);
-          acc = mma(kh, qh[ks], acc);
-          acc = mma(kl, qh[ks], acc);
-          acc = mma(kh, ql[ks], acc);
-        }
+    for (int ks = 0; ks < KS; ++ks) {
+      bf16x8 kh[4], kl[4];
 #pragma unroll
-        for (int j = 0; j < 4; ++j) {
-          const int dt = (w - jt) * 16 + l15 - quad * 4 - j;
-          acc[j] = dt >= 0 ? acc[j] * pw(dt) : 0.f;
-        }
+      for (int jt = 0; jt < 4; ++jt) {
+        const int at = swz(jt * 16 + l15, ks * 32 + quad * 8, DP);
+        kh[jt] = *reinterpret_cast<const bf16x8*>(Kh + at);
+        kl[jt] = *reinterpret_cast<const bf16x8*>(Kl + at);
       }
-      p[jt] = acc;
+#pragma unroll
+      for (int jt = 0; jt < 4; ++jt) p[jt] = mma(kh[jt], qh[ks], p[jt]);
+#pragma unroll
+      for (int jt = 0; jt < 4; ++jt) p[jt] = mma(kl[jt], qh[ks], p[jt]);
+#pragma unroll
+      for (int jt = 0; jt < 4; ++jt) p[jt] = mma(kh[jt], ql[ks], p[jt]);
     }
+#pragma unroll
+    for (int jt = 0; jt < 4; ++jt)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int dt = (w - jt) * 16 + l15 - quad * 4 - j;
+        p[jt][j] = dt >= 0 ? p[jt][j] * pw(dt) : 0.f;
+      }
     // what the earlier chunks' state gives, then this chunk's own tokens
     floatx4 o[NT4];
 #pragma unroll
-    for (int nt = 0; nt < NT4; ++nt) {
-      o[nt] = (floatx4){0.f, 0.f, 0.f, 0.f};
+    for (int nt = 0; nt < NT4; ++nt) o[nt] = (floatx4){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int ks = 0; ks < KS; ++ks) {
+    for (int ks = 0; ks < KS; ++ks) {
+      bf16x8 sh[NT4], sl[NT4];
+#pragma unroll
+      for (int nt = 0; nt < NT4; ++nt) {
         const int at = swz(nt * 16 + l15, ks * 32 + quad * 8, DP);
-        const bf16x8 sh = *reinterpret_cast<const bf16x8*>(Sh + at);
-        const bf16x8 sl = *reinterpret_cast<const bf16x8*>(Sl + at);
-        o[nt] = mma(qh[ks], sh, o[nt]);
-        o[nt] = mma(ql[ks], sh, o[nt]);
-        o[nt] = mma(qh[ks], sl, o[nt]);
+        sh[nt] = *reinterpret_cast<const bf16x8*>(Sh + at);
+        sl[nt] = *reinterpret_cast<const bf16x8*>(Sl + at);
       }
+#pragma unroll
+      for (int nt = 0; nt < NT4; ++nt) o[nt] = mma(qh[ks], sh[nt], o[nt]);
+#pragma unroll
+      for (int nt = 0; nt < NT4; ++nt) o[nt] = mma(ql[ks], sh[nt], o[nt]);
+#pragma unroll
+      for (int nt = 0; nt < NT4; ++nt) o[nt] = mma(qh[ks], sl[nt], o[nt]);
     }
     float f[4];
 #pragma unroll

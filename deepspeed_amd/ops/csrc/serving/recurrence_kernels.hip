@@ -355,8 +355,13 @@ __global__ __launch_bounds__(NT) void diagonal_scan_short_k(
 // gates, state update and gated read-out of one block of channels of up to 16
 // sequences in one workgroup (it owns the block's channels: nobody else reads
 // or shifts their tails). proj row = [ y (W) | x (W) ].
-constexpr int RS_W = 8;  // waves
+constexpr int RS_W = 16;  // waves
+constexpr int RS_K = 6;   // 32-wide input steps whose weights are fetched ahead
+constexpr int RS_U = 2;   // channels of a thread whose loads are issued together
 
+// TAPS > 0: that many taps, a channel's tail in registers; 0: any number.
+// VEC: n a multiple of 8 (rows of the weights start 16-byte aligned).
+template <int TAPS, bool VEC>
 __global__ __launch_bounds__(64 * RS_W) void rglru_step_k(
     const bf16* __restrict__ proj, int ld_proj, const bf16* __restrict__ cw,
     const float* __restrict__ cb, bf16* __restrict__ tail, int64_t tail_stride, int taps,
@@ -364,76 +369,151 @@ __global__ __launch_bounds__(64 * RS_W) void rglru_step_k(
     const float* __restrict__ bi, const float* __restrict__ lam, float* __restrict__ state,
     const int* __restrict__ seq_slot, const int* __restrict__ seq_start, bf16* __restrict__ out,
     int nseq, int n, int W, float c) {
+  typedef __attribute__((ext_vector_type(8))) __bf16 frag;
   extern __shared__ __attribute__((aligned(16))) char smem[];
+  __shared__ int s_slot[16], s_pos[16];
   bf16* sU = reinterpret_cast<bf16*>(smem);  // [16][pitch]
   const int pitch = (n + 31) / 32 * 32 + 8;
   const int t0 = blockIdx.x * 16, blk = blockIdx.y;
+  const int nt = min(16, nseq - t0);
   const int kept = taps - 1;
-  for (int i = threadIdx.x; i < 16 * pitch; i += 64 * RS_W) {
-    const int tk = i / pitch, k = i - tk * pitch;
-    const int t = t0 + tk;
-    float u = 0.f;
-    if (k < n && t < nseq) {
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int l15 = lane & 15, quad = lane >> 4;
+  if (threadIdx.x < 16) {
+    const int t = t0 + min((int)threadIdx.x, nt - 1);
+    s_slot[threadIdx.x] = seq_slot[t];
+    s_pos[threadIdx.x] = seq_start[t];
+  }
+  // this wave's first tile of both weights: in flight over the convolution
+  auto get = [&](const bf16* base, int o, int k) {
+    const short* row = reinterpret_cast<const short*>(base) + ((int64_t)blk * n + o) * n;
+    short8 x = {0, 0, 0, 0, 0, 0, 0, 0};
+    if (o < n) {
+      if (VEC) {
+        if (k < n) x = *reinterpret_cast<const short8*>(row + k);
+      } else {
+#pragma unroll
+        for (int e = 0; e < 8; ++e)
+          if (k + e < n) x[e] = row[k + e];
+      }
+    }
+    return x;
+  };
+  short8 pr[RS_K], pi[RS_K];
+#pragma unroll
+  for (int i = 0; i < (VEC ? RS_K : 0); ++i) {
+    pr[i] = get(wr, wave * 16 + l15, i * 32 + quad * 8);
+    pi[i] = get(wi, wave * 16 + l15, i * 32 + quad * 8);
+  }
+  for (int i = nt * pitch + threadIdx.x; i < 16 * pitch; i += 64 * RS_W) st(sU + i, 0.f);
+  for (int i = threadIdx.x; i < nt * (pitch - n); i += 64 * RS_W) {
+    const int tk = i / (pitch - n);
+    st(sU + tk * pitch + n + i - tk * (pitch - n), 0.f);
+  }
+  __syncthreads();
+  // what the wave's first tile needs at its end, in flight over the rest
+  float pS[4], pz[4], prate, pcr, pci;
+  {
+    const int ch = blk * n + min(wave * 16 + l15, n - 1);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int tk = min(quad * 4 + e, nt - 1);
+      pS[e] = state[(int64_t)s_slot[tk] * W + ch];
+      pz[e] = ld(proj + (int64_t)(t0 + tk) * ld_proj + ch);
+    }
+    prate = lam[ch];
+    pcr = br[ch];
+    pci = bi[ch];
+  }
+  if (TAPS > 0) {
+    constexpr int K = TAPS > 1 ? TAPS - 1 : 1;
+    for (int i0 = threadIdx.x; i0 < nt * n; i0 += 64 * RS_W * RS_U) {
+      float x[RS_U], cbv[RS_U], wv[RS_U][K + 1], tv[RS_U][K];
+#pragma unroll
+      for (int q = 0; q < RS_U; ++q) {
+        const int i = min(i0 + q * 64 * RS_W, nt * n - 1);
+        const int tk = i / n, ch = blk * n + i - tk * n;
+        x[q] = ld(proj + (int64_t)(t0 + tk) * ld_proj + W + ch);
+        cbv[q] = cb[ch];
+#pragma unroll
+        for (int j = 0; j < TAPS; ++j) wv[q][j] = ld(cw + (int64_t)ch * TAPS + j);
+#pragma unroll
+        for (int j = 0; j + 1 < TAPS; ++j)
+          tv[q][j] = ld(tail + (int64_t)s_slot[tk] * tail_stride + (int64_t)j * W + ch);
+      }
+#pragma unroll
+      for (int q = 0; q < RS_U; ++q) {
+        const int i = i0 + q * 64 * RS_W;
+        if (i >= nt * n) break;
+        const int tk = i / n, ch = blk * n + i - tk * n;
+        float u = wv[q][TAPS > 0 ? TAPS - 1 : 0] * x[q];
+#pragma unroll
+        for (int j = 1; j < TAPS; ++j)
+          if (s_pos[tk] - j >= 0) u += wv[q][TAPS - 1 - j] * tv[q][TAPS - 1 - j];
+        st(sU + tk * pitch + i - tk * n, u + cbv[q]);
+        bf16* tl = tail + (int64_t)s_slot[tk] * tail_stride + ch;
+#pragma unroll
+        for (int j = 0; j + 1 < TAPS; ++j)
+          st(tl + (int64_t)j * W, j + 2 < TAPS ? tv[q][j + 1 < K ? j + 1 : 0] : x[q]);
+      }
+    }
+  } else {
+    for (int i = threadIdx.x; i < nt * n; i += 64 * RS_W) {
+      const int tk = i / n, k = i - tk * n;
       const int ch = blk * n + k;
-      const bf16 xin = proj[(int64_t)t * ld_proj + W + ch];
-      const int pos = seq_start[t];
-      bf16* tl = tail + (int64_t)seq_slot[t] * tail_stride + ch;
+      const bf16 xin = proj[(int64_t)(t0 + tk) * ld_proj + W + ch];
+      bf16* tl = tail + (int64_t)s_slot[tk] * tail_stride + ch;
       const bf16* w = cw + (int64_t)ch * taps;
-      u = ld(w + kept) * ld(&xin);
+      float u = ld(w + kept) * ld(&xin);
       for (int j = 1; j <= kept; ++j)
-        if (pos - j >= 0) u += ld(w + kept - j) * ld(tl + (int64_t)(kept - j) * W);
-      u += cb[ch];
+        if (s_pos[tk] - j >= 0) u += ld(w + kept - j) * ld(tl + (int64_t)(kept - j) * W);
+      st(sU + tk * pitch + k, u + cb[ch]);
       for (int j = 0; j + 1 < kept; ++j) tl[(int64_t)j * W] = tl[(int64_t)(j + 1) * W];
       if (kept > 0) tl[(int64_t)(kept - 1) * W] = xin;
     }
-    st(sU + i, u);
   }
   __syncthreads();
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  const int l15 = lane & 15, quad = lane >> 4;
-  const bool vec = (n & 7) == 0;
   for (int ot = wave; ot * 16 < n; ot += RS_W) {
     const int o = ot * 16 + l15;
-    const short* rr = reinterpret_cast<const short*>(wr) + ((int64_t)blk * n + o) * n;
-    const short* ri = reinterpret_cast<const short*>(wi) + ((int64_t)blk * n + o) * n;
-    auto get = [&](const short* row, int k) {
-      short8 x = {0, 0, 0, 0, 0, 0, 0, 0};
-      if (o < n) {
-        if (vec) {
-          if (k < n) x = *reinterpret_cast<const short8*>(row + k);
-        } else {
+    const int ch = blk * n + min(o, n - 1);
+    if (ot != wave) {
 #pragma unroll
-          for (int e = 0; e < 8; ++e)
-            if (k + e < n) x[e] = row[k + e];
-        }
+      for (int e = 0; e < 4; ++e) {
+        const int tk = min(quad * 4 + e, nt - 1);
+        pS[e] = state[(int64_t)s_slot[tk] * W + ch];
+        pz[e] = ld(proj + (int64_t)(t0 + tk) * ld_proj + ch);
       }
-      return x;
-    };
-    typedef __attribute__((ext_vector_type(8))) __bf16 frag;
-    floatx4 ar = {0.f, 0.f, 0.f, 0.f}, ai = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
-    for (int kk = 0; kk < n; kk += 32) {
-      const int k = kk + quad * 8;
-      const frag fa = *reinterpret_cast<const frag*>(sU + l15 * pitch + k);
-      ar = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fa, __builtin_bit_cast(frag, get(rr, k)), ar, 0,
-                                                   0, 0);
-      ai = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fa, __builtin_bit_cast(frag, get(ri, k)), ai, 0,
-                                                   0, 0);
+      prate = lam[ch];
+      pcr = br[ch];
+      pci = bi[ch];
     }
+    floatx4 ar = {0.f, 0.f, 0.f, 0.f}, ai = {0.f, 0.f, 0.f, 0.f};
+    auto step = [&](int kk, short8 r, short8 i) {
+      const frag fa = *reinterpret_cast<const frag*>(sU + l15 * pitch + kk + quad * 8);
+      ar = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fa, __builtin_bit_cast(frag, r), ar, 0, 0, 0);
+      ai = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fa, __builtin_bit_cast(frag, i), ai, 0, 0, 0);
+    };
+    int k0 = 0;
+    if (VEC && ot == wave) {
+#pragma unroll
+      for (int i = 0; i < RS_K; ++i)
+        if (i * 32 < n) step(i * 32, pr[i], pi[i]);
+      k0 = RS_K * 32;
+    }
+#pragma unroll 2
+    for (int kk = k0; kk < n; kk += 32)
+      step(kk, get(wr, o, kk + quad * 8), get(wi, o, kk + quad * 8));
     if (o >= n) continue;
-    const int ch = blk * n + o;
-    const float rate = c * softplus_(lam[ch]), cr = br[ch], ci = bi[ch];
+    const float rate = c * softplus_(prate);
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
-      const int t = t0 + quad * 4 + e;
-      if (t < nseq) {
+      const int tk = quad * 4 + e;
+      if (tk < nt) {
         float a, b;
-        rglru_pair<false>(ar[e] + cr, ai[e] + ci, ld(sU + (quad * 4 + e) * pitch + o), rate, a, b);
-        float* Sg = state + (int64_t)seq_slot[t] * W + ch;
-        const float S = a * *Sg + b;
-        *Sg = S;
-        st(out + (int64_t)t * W + ch,
-           S * gate_act<false>(ld(proj + (int64_t)t * ld_proj + ch), 0));
+        rglru_pair<false>(ar[e] + pcr, ai[e] + pci, ld(sU + tk * pitch + o), rate, a, b);
+        const float Sn = a * pS[e] + b;
+        state[(int64_t)s_slot[tk] * W + ch] = Sn;
+        st(out + (int64_t)(t0 + tk) * W + ch, Sn * gate_act<false>(pz[e], 0));
       }
     }
   }
@@ -487,12 +567,23 @@ __global__ __launch_bounds__(RT_T) void retention_step_k(
     float acc = 0.f;
     if (c < vdim) {
       const float vc = ld(v + (int64_t)t * ld_v + h * vdim + c);
-#pragma unroll 8
-      for (int d = rg; d < dim; d += RG) {
-        float* p = Sh + (int64_t)d * vdim + c;
-        const float S = g * *p + sk[d] * vc;
-        *p = S;
-        acc += sq[d] * S;
+      // eight rows at a time: all loads before the first store
+      for (int d0 = rg; d0 < dim; d0 += 8 * RG) {
+        float S[8];
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+          const int d = d0 + i * RG;
+          S[i] = d < dim ? Sh[(int64_t)d * vdim + c] : 0.f;
+        }
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+          const int d = d0 + i * RG;
+          if (d < dim) {
+            S[i] = g * S[i] + sk[d] * vc;
+            Sh[(int64_t)d * vdim + c] = S[i];
+            acc += sq[d] * S[i];
+          }
+        }
       }
     }
     sp[threadIdx.x] = acc;
@@ -950,10 +1041,17 @@ int dsv_rglru_step(const void* proj, int ld_proj, const void* cw, const float* c
   if ((uintptr_t)wr % 16 || (uintptr_t)wi % 16) return -2;
   const size_t lds = (size_t)16 * ((n + 31) / 32 * 32 + 8) * 2;
   if (lds > 48 * 1024) return -3;
-  rglru_step_k<<<dim3((nseq + 15) / 16, blocks), 64 * RS_W, lds, s>>>(
-      (const bf16*)proj, ld_proj, (const bf16*)cw, cb, (bf16*)tail, tail_stride, taps,
-      (const bf16*)wr, (const bf16*)wi, br, bi, lam, state, seq_slot, seq_start, (bf16*)out, nseq,
-      n, blocks * n, c);
+#define RGSTEP(TAPS, VEC)                                                                       \
+  rglru_step_k<TAPS, VEC><<<dim3((nseq + 15) / 16, blocks), 64 * RS_W, lds, s>>>(                \
+      (const bf16*)proj, ld_proj, (const bf16*)cw, cb, (bf16*)tail, tail_stride, taps,          \
+      (const bf16*)wr, (const bf16*)wi, br, bi, lam, state, seq_slot, seq_start, (bf16*)out,    \
+      nseq, n, blocks * n, c)
+  if (n % 8) RGSTEP(0, false);
+  else if (taps == 4) RGSTEP(4, true);
+  else if (taps == 3) RGSTEP(3, true);
+  else if (taps == 2) RGSTEP(2, true);
+  else RGSTEP(0, true);
+#undef RGSTEP
   return (int)hipGetLastError();
 }
 

@@ -1131,8 +1131,8 @@ def test_scan_with_a_fixed_decay_against_eager(H, d, dv, vdt, monkeypatch):
 
 @pytest.mark.gpu
 @pytest.mark.parametrize("blocks,n,taps,N", [
-    (3, 5, 4, 3), (2, 72, 4, 1), (1, 20, 1, 5), (4, 64, 2, 17), (2, 256, 4, 40),
-    (1, 200, 7, 2)])
+    (3, 5, 4, 3), (2, 72, 3, 1), (1, 20, 1, 5), (4, 64, 2, 17), (2, 256, 4, 40),
+    (1, 200, 7, 2), (1, 328, 4, 5)])
 def test_single_token_recurrence_step_against_its_parts(blocks, n, taps, N,
                                                         monkeypatch):
     """One fused kernel against convolution, gates and scan one by one, over

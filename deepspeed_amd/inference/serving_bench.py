@@ -1328,11 +1328,22 @@ def _redudra_kernel_rows(z, dev):
                 n * W * 26 + 4 * W * (W // nbk))
         bc = (torch.randn(n, 2 * SN, device=dev) * 0.1).to(bf)
         so = torch.empty(n, W, device=dev, dtype=bf)
-        row("selective_scan (savovik), " + case, "",
-            lambda: sk.selective_scan(u, a, zero, a_log, bc[:, :SN],
-                                      bc[:, SN:], zero, pin[:, :W],
-                                      rc.states["sel"], bt, 1.0, so),
-            n * W * 10 + n * 2 * SN * 2 + 2 * NB * W * SN * 4)
+
+        def sel():
+            sk.selective_scan(u, a, zero, a_log, bc[:, :SN], bc[:, SN:],
+                              zero, pin[:, :W], rc.states["sel"], bt, 1.0,
+                              so)
+
+        def conv_sel():
+            conv_silu_ragged(pin[:, W:], cw, rc.states["conv"], bt, zero, bf)
+            sel()
+
+        sel_bytes = n * W * 10 + n * 2 * SN * 2 + 2 * NB * W * SN * 4
+        if cnt > 1:
+            row("selective_scan (savovik), " + case, "", sel, sel_bytes)
+        else:       # the step kernel holds the convolution as well
+            row("conv_silu + selective_scan (savovik), " + case, "",
+                conv_sel, sel_bytes + n * W * 18)
         rc.end_step()
         del rc, pin, u, a
     gu = torch.randn(T, 2 * F, device=dev).to(bf)

@@ -14,6 +14,7 @@ from .fizesun import FizesunConfig, FizesunForCausalLM, fizesun_tiny
 from .savovik import SavovikConfig, SavovikForCausalLM, savovik_tiny
 from .numolorn import NumolornConfig, NumolornForCausalLM, numolorn_tiny
 from .redudra import RedudraConfig, RedudraForCausalLM, redudra_tiny
+from .fubolix import FubolixConfig, FubolixForCausalLM, fubolix_tiny
 from .registry import (architectures, build_model, load_pretrained,
                        register_architecture)
 
@@ -30,6 +31,7 @@ __all__ = [
     "SavovikConfig", "SavovikForCausalLM", "savovik_tiny",
     "NumolornConfig", "NumolornForCausalLM", "numolorn_tiny",
     "RedudraConfig", "RedudraForCausalLM", "redudra_tiny",
+    "FubolixConfig", "FubolixForCausalLM", "fubolix_tiny",
     "architectures", "build_model", "load_pretrained",
     "register_architecture",
 ]

@@ -89,6 +89,7 @@ def _dataclass_builder(config_cls, model_cls, rename=None):
 
 def _register_builtin():
     from .fizesun import FizesunConfig, FizesunForCausalLM
+    from .fubolix import build_from_config as build_fubolix
     from .llama import LlamaConfig, LlamaForCausalLM
     from .lolulorn import build_from_config as build_lolulorn
     from .mixtral import MixtralConfig, MixtralForCausalLM
@@ -114,6 +115,7 @@ def _register_builtin():
     register_architecture("Savovik", build_savovik)
     register_architecture("Numolorn", build_numolorn, wants_tensors=True)
     register_architecture("Redudra", build_redudra)
+    register_architecture("Fubolix", build_fubolix)
 
 
 _register_builtin()

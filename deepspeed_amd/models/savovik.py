@@ -42,7 +42,7 @@ from ..ops.activations import act_rows
 from ..ops.causal_conv import conv_silu_ragged
 from ..ops.linear_recurrence import gate_group_norm, linear_scan, ssd_prep
 from ..ops.norms import embed_rows, gated_add_, rms_norm_rows
-from ..ops.rope import rope_tables
+from ..ops.rope import rope_tables, temperature_table
 from ..ops.selective_scan import selective_scan
 from ..ops.window_attention import attn_prep, window_attention
 
@@ -135,13 +135,18 @@ def rot_tables(rot, max_seq, device):
 
 
 class GroupedAttention(nn.Module):
-    """Grouped-query attention over paged rows; what differs between its two
-    uses is given by flags: projection biases, per-head query/key norms, the
-    rotary pairing, unit-RMS values, the score cap and the kind of mask (a
-    window may keep a sequence's first tokens)."""
+    """Grouped-query attention over paged rows; what differs between its uses
+    is given by flags: projection biases, query/key norms ("head": per head
+    with a weight, "after": unit RMS after the rotation), the rotary pairing,
+    unit-RMS values, the score cap, the kind of mask (a window may keep a
+    sequence's first tokens; None: causal), a short convolution over the
+    projected channels, keys as values, queries scaled by position, a score
+    without key in the softmax ("learned" per head, "one": zero) and a gate
+    per head."""
 
-    def __init__(self, m: dict, eps, dtype, *, bias, qk_norm, layout, v_unit,
-                 mask):
+    def __init__(self, m: dict, eps, dtype, *, bias=False, qk_norm=None,
+                 layout="half", v_unit=False, mask=None, conv=False,
+                 v_from_k=False, q_temp=False, sink=None, gate=False):
         super().__init__()
         self.heads = int(m["heads"])
         self.kv_heads = int(m.get("kv_heads", self.heads))
@@ -152,42 +157,76 @@ class GroupedAttention(nn.Module):
                 self.rot_dims > self.dim:
             raise ValueError("attention: heads must be a multiple of kv_heads "
                              "and rot.dims even and at most dim")
+        if v_from_k and self.vdim != self.dim:
+            raise ValueError("attention: keys as values need vdim == dim")
         self.scale = float(m["scale"])
         self.softcap = float(m.get("softcap") or 0.0)
         size = int((m.get("mask") or {}).get("size", 0))
-        self.keep_first = int((m.get("mask") or {}).get("keep_first", 0))
+        self.keep_first = int((m.get("mask") or {}).get("keep_first", 0)) \
+            if mask else 0
         self.window = size if mask == "window" else 0
         self.chunk = size if mask == "chunk" else 0
         self.layout = layout
-        self.norm = "head" if qk_norm else None
+        self.norm = {True: "head", False: None}.get(qk_norm, qk_norm)
         self.v_unit_eps = eps if v_unit else None
         self.eps = eps
         self.has_bias = bias
-        self.n_in = self.heads * self.dim + self.kv_heads * (self.dim
-                                                             + self.vdim)
+        self.v_from_k = v_from_k
+        self.n_in = self.heads * self.dim + self.kv_heads * (
+            self.dim + (0 if v_from_k else self.vdim))
         self.n_out = self.heads * self.vdim
-        self.q_norm = _w(self.dim, dtype=torch.float32) if qk_norm else None
-        self.k_norm = _w(self.dim, dtype=torch.float32) if qk_norm else None
+        weighted = self.norm == "head"
+        self.q_norm = _w(self.dim, dtype=torch.float32) if weighted else None
+        self.k_norm = _w(self.dim, dtype=torch.float32) if weighted else None
+        self.taps = int(m.get("conv", 1)) if conv else 0
+        if conv and self.taps < 1:
+            raise ValueError("attention: a convolution has at least one tap")
+        self.conv = _w(self.n_in, self.taps, dtype=dtype) if conv else None
+        temp = m.get("q_temp") if q_temp else None
+        self.q_temp = None
+        if temp:
+            every = temp["every"]
+            self.q_temp = (float(temp["coef"]), every)
+            if not every > 0:
+                raise ValueError("attention: q_temp.every must be positive")
+        if sink == "one":
+            self.register_buffer("sink", torch.zeros(
+                self.heads, dtype=torch.float32), persistent=False)
+        else:
+            self.sink = _w(self.heads, dtype=torch.float32) \
+                if sink == "learned" else None
+        self.has_gate = gate
 
     @property
     def row_dim(self):
         return self.kv_heads * (self.dim + self.vdim)
 
+    def state_shapes(self, dtype):
+        return {"conv": ((self.taps - 1, self.n_in), dtype)} \
+            if self.taps else {}
+
     def run(self, proj, cache: PagedStateCache, stream, out=None,
-            out_scale=1.0):
-        """proj: this step's q|k|v (a column slice is fine). Returns the
-        heads' results side by side, before the output projection."""
+            out_scale=1.0, states=None, gate=None, side=None):
+        """proj: this step's q|k|v (a column slice is fine); ``gate`` the
+        heads' gate pre-activations; ``side`` = (z, out, act), an activation
+        done beside the prologue. Returns the heads' results side by side,
+        before the output projection."""
         b = cache.batch
         cos, sin = rot_tables(self.rot, cache.max_seq, proj.device) \
             if self.rot_dims else (None, None)
+        factor = temperature_table(cache.max_seq, *self.q_temp, proj.device) \
+            if self.q_temp else None
         pool = cache.pools[stream]
         q = attn_prep(proj, b, pool, self.q_norm, self.k_norm, self.eps,
                       self.heads, self.kv_heads, self.dim, self.vdim,
                       self.rot_dims, cos, sin, True, self.norm, self.layout,
-                      self.v_unit_eps)
+                      self.v_unit_eps,
+                      (self.conv, states["conv"]) if self.taps else None,
+                      self.v_from_k, factor, side)
         return window_attention(q, pool, b, self.kv_heads, self.dim,
                                 self.vdim, self.scale, self.window,
-                                self.keep_first, None, self.chunk, self.softcap, out_scale, out)
+                                self.keep_first, None, self.chunk,
+                                self.softcap, out_scale, out, self.sink, gate)
 
 
 class AttentionMixer(nn.Module):

@@ -9,8 +9,9 @@
 * ``glu(gu, act)``: ``act(gate) * up`` with ``act`` "silu" or "gelu_tanh"
   (``0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3)))``), same layout.
 * ``act_rows(z, act)``: a plain activation of a projection, ``act`` one of
-  "gelu_erf" (``0.5 z (1 + erf(z / sqrt 2))``), "gelu_tanh", "silu"; ``z`` may
-  be a column slice of a wider projection.
+  "gelu_erf" (``0.5 z (1 + erf(z / sqrt 2))``), "gelu_tanh", "silu", "relu2"
+  (``max(z, 0)^2``); ``z`` may be a column slice of a wider projection, ``out``
+  one of a wider buffer.
 * ``softcap_rows(z, cap)``: ``cap * tanh(z / cap)``, returned in fp32.
 All evaluate in fp32 and round once.
 """
@@ -64,23 +65,27 @@ def glu(gu, act):
     return (a * u).to(gu.dtype)
 
 
-ROW_ACTS = ("gelu_erf", "gelu_tanh", "silu")
+ROW_ACTS = ("gelu_erf", "gelu_tanh", "silu", "relu2")
 
 
-def act_rows(z, act):
-    """z [T, F] (rows contiguous, any row stride) -> act(z), contiguous."""
+def act_rows(z, act, out=None):
+    """z [T, F] (rows contiguous, any row stride) -> act(z), contiguous or in
+    ``out`` ([T, F] in z's dtype, rows contiguous)."""
     if act not in ROW_ACTS:
         raise ValueError(f"unknown activation {act!r}")
     if z.is_cuda and _sk().enabled():
-        return _sk().act_rows(z, ROW_ACTS.index(act))
+        return _sk().act_rows(z, ROW_ACTS.index(act), out)
     zf = z.float()
     if act == "gelu_erf":
         y = F.gelu(zf)
     elif act == "gelu_tanh":
         y = F.gelu(zf, approximate="tanh")
-    else:
+    elif act == "silu":
         y = F.silu(zf)
-    return y.to(z.dtype)
+    else:
+        y = F.relu(zf).square()
+    y = y.to(z.dtype)
+    return y if out is None else out.copy_(y)
 
 
 def softcap_rows(z, cap):

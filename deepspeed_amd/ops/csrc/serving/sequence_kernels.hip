@@ -155,9 +155,23 @@ __global__ __launch_bounds__(NT) void attn_prep_vec_k(
 // window), n_keep = min(keep_first, lo). They are walked as one virtual range
 // in chunks of KC, staged through LDS; scores, online softmax and the
 // weighted sum are float. With nsplit > 1 the block writes (max, sum,
-// unnormalised sum) and window_attn_merge_k finishes.
+// unnormalised sum) and window_attn_merge_k finishes. `sink` (one score per
+// query head, or null) joins the denominator as exp(sink) without a value;
+// `gate` (pre-activations, row stride ld_gate, or null) scales head h by
+// sigmoid(gate[t, h]).
 constexpr int WHG = 8;
 constexpr int WVPT = 2;  // value columns per thread: vdim <= WVPT * NT
+
+// factor on a head's unnormalised sum: l = sum of exp(score - m)
+template <typename T>
+__device__ __forceinline__ float head_factor(float l, float m, int t, int h, float out_scale,
+                                             const float* __restrict__ sink,
+                                             const T* __restrict__ gate, int ld_gate) {
+  if (sink) l += expf(sink[h] - m);  // inf where the sink dwarfs every score: weight zero
+  float f = out_scale / l;
+  if (gate) f *= sigmoidf_(ld(gate + (int64_t)t * ld_gate + h));
+  return f;
+}
 
 template <typename T>
 __global__ __launch_bounds__(NT) void window_attn_k(
@@ -168,7 +182,8 @@ __global__ __launch_bounds__(NT) void window_attn_k(
     T* __restrict__ out,       // [Ttok, H, vdim]
     float* __restrict__ part,  // [Ttok, nsplit, H, vdim + 2] when nsplit > 1
     int ld_out, int H, int G, int dim, int vdim, int KC, int nsplit, float scale, int window,
-    int keep_first, int chunk, float softcap, float out_scale) {
+    int keep_first, int chunk, float softcap, float out_scale, const float* __restrict__ sink,
+    const T* __restrict__ gate, int ld_gate) {
   extern __shared__ float smem[];
   const int DS = dim | 1;
   float* qs = smem;              // [WHG][dim]
@@ -290,7 +305,8 @@ __global__ __launch_bounds__(NT) void window_attn_k(
     for (int h = 0; h < WHG; ++h) {
       if (h < nh) {
         if (nsplit == 1) {
-          const float inv = out_scale / lrun[h];
+          const float inv =
+              head_factor(lrun[h], mrun[h], t, hbase + h, out_scale, sink, gate, ld_gate);
 #pragma unroll
           for (int i = 0; i < WVPT; ++i) {
             const int col = tid + i * NT;
@@ -317,7 +333,8 @@ __global__ __launch_bounds__(NT) void window_attn_k(
 template <typename T>
 __global__ __launch_bounds__(NT) void window_attn_merge_k(
     const float* __restrict__ part, T* __restrict__ out, int ld_out, int H, int vdim,
-    int nsplit, float out_scale) {
+    int nsplit, float out_scale, const float* __restrict__ sink, const T* __restrict__ gate,
+    int ld_gate) {
   const int t = blockIdx.x, h = blockIdx.y;
   float m = -INFINITY;
   for (int s = 0; s < nsplit; ++s) {
@@ -329,13 +346,14 @@ __global__ __launch_bounds__(NT) void window_attn_merge_k(
     const float* pp = part + (((int64_t)t * nsplit + s) * H + h) * (vdim + 2);
     if (pp[1] > 0.f) l += pp[1] * expf(pp[0] - m);
   }
+  const float f = head_factor(l, m, t, h, out_scale, sink, gate, ld_gate);
   for (int c = threadIdx.x; c < vdim; c += NT) {
     float a = 0.f;
     for (int s = 0; s < nsplit; ++s) {
       const float* pp = part + (((int64_t)t * nsplit + s) * H + h) * (vdim + 2);
       if (pp[1] > 0.f) a += pp[2 + c] * expf(pp[0] - m);
     }
-    st(out + (int64_t)t * ld_out + h * vdim + c, a / l * out_scale);
+    st(out + (int64_t)t * ld_out + h * vdim + c, a * f);
   }
 }
 
@@ -387,7 +405,8 @@ __global__ __launch_bounds__(256, (DKT_MAX <= 8 ? 2 : 1)) void window_attn_mfma_
     const int* __restrict__ table, int maxb, int bs, bf16* __restrict__ out, int ld_out,
     float* __restrict__ part,  // [Ttok, nsplit, H, vdim + 2] when nsplit > 1
     int H, int G, int dim, int vdim, int nsplit, float scale, int window, int keep_first,
-    int chunk, float softcap, float out_scale) {
+    int chunk, float softcap, float out_scale, const float* __restrict__ sink,
+    const bf16* __restrict__ gate, int ld_gate) {
   extern __shared__ __attribute__((aligned(16))) char smem_raw[];
   constexpr int CPT = (2 * DKT_MAX + 4 * DVB + 7) / 8;  // 16-byte chunks per thread and tile
   const int dimP = (dim + 15) & ~15;
@@ -663,7 +682,7 @@ __global__ __launch_bounds__(256, (DKT_MAX <= 8 ? 2 : 1)) void window_attn_mfma_
           if (d < vdim) pp[2 + d] = oacc[db][r];
         }
     } else {
-      const float inv = out_scale / lrun;
+      const float inv = head_factor(lrun, mrun, t, h, out_scale, sink, gate, ld_gate);
       bf16* o = out + (int64_t)t * ld_out + h * vdim;
 #pragma unroll
       for (int db = 0; db < DVB; ++db)
@@ -682,7 +701,7 @@ int launch_window_attn_mfma(const void* q, const void* pool, const int* work, in
                             int bs, void* out, int ld_out, float* part, int Ttok, int H, int G,
                             int dim, int vdim, int nsplit, float scale, int window,
                             int keep_first, int chunk, float softcap, float out_scale,
-                            hipStream_t s) {
+                            const float* sink, const void* gate, int ld_gate, hipStream_t s) {
   const int dimP = (dim + 15) & ~15;
   const size_t lds = ((size_t)TB_KEYS * (dimP + 8) * 2 + (size_t)DVB * 32 * VT_STRIDE * 2) *
                      (PREFETCH ? 2 : 1);
@@ -690,10 +709,11 @@ int launch_window_attn_mfma(const void* q, const void* pool, const int* work, in
   kern<<<dim3(nwork, nsplit), 256, lds, s>>>((const short*)q, (const short*)pool, work, cu,
                                              seq_start, table, maxb, bs, (bf16*)out, ld_out,
                                              part, H, G, dim, vdim, nsplit, scale, window,
-                                             keep_first, chunk, softcap, out_scale);
+                                             keep_first, chunk, softcap, out_scale, sink,
+                                             (const bf16*)gate, ld_gate);
   if (nsplit > 1)
-    window_attn_merge_k<bf16><<<dim3(Ttok, H), NT, 0, s>>>(part, (bf16*)out, ld_out, H, vdim,
-                                                           nsplit, out_scale);
+    window_attn_merge_k<bf16><<<dim3(Ttok, H), NT, 0, s>>>(
+        part, (bf16*)out, ld_out, H, vdim, nsplit, out_scale, sink, (const bf16*)gate, ld_gate);
   return (int)hipGetLastError();
 }
 
@@ -1290,65 +1310,84 @@ __global__ __launch_bounds__(NT) void retention_prep_k(
 
 // ------------------------------------- attention prologue, per-head options
 // proj row (stride ld_proj) = [ q (H x dim) | k (G x dim) | v (G x vdim) ].
-// NORM: 0 none, 2 per head over dim with one weight of size dim shared by the
-// heads. Rotation of the first rot_dims coordinates of each head, pairing
-// (2i, 2i+1) (HALF false) or (i, i + rot_dims/2) (HALF true). v_eps >= 0:
-// every value head is divided by its root mean square. One wave per head.
-template <typename T, bool HALF>
-__global__ __launch_bounds__(NT) void attn_prep_heads_k(
-    const T* __restrict__ proj, int ld_proj, const float* __restrict__ wq,
-    const float* __restrict__ wk, const int* __restrict__ tok_pos,
-    const int* __restrict__ tok_row, const float* __restrict__ cosT,
-    const float* __restrict__ sinT, T* __restrict__ pool, T* __restrict__ q_out, int H, int G,
-    int dim, int vdim, int rot_dims, int own_kv, int norm, float eps, float v_eps) {
+// norm: 0 none, 2 per head over dim with one weight of size dim shared by the
+// heads, 3 per head without weight AFTER the rotation. Rotation of the first
+// rot_dims coordinates of each head, pairing (2i, 2i+1) or, with half, (i, i +
+// rot_dims/2). qfac (one factor per position, or null) multiplies the finished
+// queries. v_eps >= 0: every value head is divided by its root mean square;
+// v_from_k: the values are the projected keys themselves (no v columns, vdim =
+// dim). One wave per head.
+struct PrepArgs {
+  int ld_proj, H, G, dim, vdim, rot_dims, own_kv, norm, half, v_from_k;
+  float eps, v_eps;
+  const float *wq, *wk, *cosT, *sinT, *qfac;
+  const int *tok_pos, *tok_row;
+};
+
+template <typename T>
+__global__ __launch_bounds__(NT) void attn_prep_heads_k(const T* __restrict__ proj,
+                                                        T* __restrict__ pool,
+                                                        T* __restrict__ q_out, PrepArgs a) {
   const int t = blockIdx.x;
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
-  const T* p = proj + (int64_t)t * ld_proj;
+  const T* p = proj + (int64_t)t * a.ld_proj;
+  const int dim = a.dim, vdim = a.vdim, H = a.H, G = a.G, rot_dims = a.rot_dims;
   const int nq = H * dim, nk = G * dim, nv = G * vdim;
   const int half = rot_dims >> 1;
-  const float* cs = cosT + (int64_t)tok_pos[t] * half;
-  const float* sn = sinT + (int64_t)tok_pos[t] * half;
-  T* row = own_kv ? pool + (int64_t)tok_row[t] * (nk + nv) : nullptr;
-  const int jobs = own_kv ? H + 2 * G : H;
+  const float* cs = a.cosT + (int64_t)a.tok_pos[t] * half;
+  const float* sn = a.sinT + (int64_t)a.tok_pos[t] * half;
+  T* row = a.own_kv ? pool + (int64_t)a.tok_row[t] * (nk + nv) : nullptr;
+  const int jobs = a.own_kv ? H + 2 * G : H;
   for (int job = wid; job < jobs; job += NT / 64) {
     if (job < H + G) {  // a query or key head
       const bool is_q = job < H;
       const T* in = is_q ? p + job * dim : p + nq + (job - H) * dim;
       T* out = is_q ? q_out + (int64_t)t * nq + job * dim : row + (job - H) * dim;
-      const float* w = is_q ? wq : wk;
+      const float* w = is_q ? a.wq : a.wk;
+      const float fac = is_q && a.qfac ? a.qfac[a.tok_pos[t]] : 1.f;
       float inv = 1.f;
-      if (norm == 2) {
+      if (a.norm == 2) {
         float ss = 0.f;
         for (int c = lane; c < dim; c += 64) {
           const float v = ld(in + c);
           ss += v * v;
         }
-        inv = rsqrtf(wave_sum(ss) / (float)dim + eps);
+        inv = rsqrtf(wave_sum(ss) / (float)dim + a.eps);
       }
-      for (int c = lane; c < dim; c += 64) {
-        float v = ld(in + c) * inv * (norm == 2 ? w[c] : 1.f);
+      auto turned = [&](int c) -> float {
+        float v = ld(in + c) * inv * (a.norm == 2 ? w[c] : 1.f);
         if (c < rot_dims) {
-          const int j = HALF ? (c < half ? c + half : c - half) : (c ^ 1);
-          const float o = ld(in + j) * inv * (norm == 2 ? w[j] : 1.f);
-          const int f = HALF ? (c < half ? c : c - half) : (c >> 1);
-          const bool second = HALF ? c >= half : (c & 1);
+          const int j = a.half ? (c < half ? c + half : c - half) : (c ^ 1);
+          const float o = ld(in + j) * inv * (a.norm == 2 ? w[j] : 1.f);
+          const int f = a.half ? (c < half ? c : c - half) : (c >> 1);
+          const bool second = a.half ? c >= half : (c & 1);
           const float co = cs[f], si = sn[f];
           v = second ? v * co + o * si : v * co - o * si;
         }
-        st(out + c, v);
+        return v;
+      };
+      float post = fac;
+      if (a.norm == 3) {
+        float ss = 0.f;
+        for (int c = lane; c < dim; c += 64) {
+          const float v = turned(c);
+          ss += v * v;
+        }
+        post *= rsqrtf(wave_sum(ss) / (float)dim + a.eps);
       }
+      for (int c = lane; c < dim; c += 64) st(out + c, turned(c) * post);
     } else {  // a value head
       const int g = job - H - G;
-      const T* in = p + nq + nk + g * vdim;
+      const T* in = a.v_from_k ? p + nq + g * dim : p + nq + nk + g * vdim;
       T* out = row + nk + g * vdim;
       float inv = 1.f;
-      if (v_eps >= 0.f) {
+      if (a.v_eps >= 0.f) {
         float ss = 0.f;
         for (int c = lane; c < vdim; c += 64) {
           const float v = ld(in + c);
           ss += v * v;
         }
-        inv = rsqrtf(wave_sum(ss) / (float)vdim + v_eps);
+        inv = rsqrtf(wave_sum(ss) / (float)vdim + a.v_eps);
       }
       for (int c = lane; c < vdim; c += 64) st(out + c, ld(in + c) * inv);
     }
@@ -1609,102 +1648,192 @@ __global__ __launch_bounds__(NT) void ssd_prep_vec_k(
 
 // The per-head prologue with eight values per lane: a head is shared by LG
 // lanes (a power of two, 8 * LG >= dim and vdim); all sizes multiples of 8.
-template <typename T, bool HALF, int LG>
+// Two more steps share the launch:
+// * TAPS > 0: a short causal convolution over every projected channel first
+//   (weights [channels, TAPS]; earlier inputs come from this step's rows, from
+//   the slot's tail, or are zero). A workgroup takes `toks` neighbouring tokens
+//   so that weights and earlier rows stay in registers from one token to the
+//   next. shift_tail: every sequence brings exactly one token, so the lane that
+//   reads a channel's tail is its only reader and moves it on in place.
+// * side: workgroups with blockIdx.y >= ny square the positive part of another
+//   column slice (the feed-forward's first product).
+template <typename T>
+struct PrepSteps {
+  const T* conv_w;
+  T* tails;
+  int64_t tail_stride;
+  const int *cu, *seq_slot, *tok_seq;
+  int shift_tail, toks, ny;
+  const T* side_in;
+  T* side_out;
+  int side_n, side_ld_in, side_ld_out;
+};
+
+template <typename T, int LG, int TAPS>
 __global__ __launch_bounds__(NT) void attn_prep_heads_vec_k(
-    const T* __restrict__ proj, int ld_proj, const float* __restrict__ wq,
-    const float* __restrict__ wk, const int* __restrict__ tok_pos,
-    const int* __restrict__ tok_row, const float* __restrict__ cosT,
-    const float* __restrict__ sinT, T* __restrict__ pool, T* __restrict__ q_out, int H, int G,
-    int dim, int vdim, int rot_dims, int own_kv, int norm, float eps, float v_eps) {
-  const int t = blockIdx.x;
+    const T* __restrict__ proj, T* __restrict__ pool, T* __restrict__ q_out, int Ttok, PrepArgs a,
+    PrepSteps<T> e) {
+  constexpr int TAIL = TAPS > 1 ? TAPS - 1 : 1;
+  const int t0 = blockIdx.x * e.toks, t1 = min(Ttok, t0 + e.toks);
+  if ((int)blockIdx.y >= e.ny) {
+    for (int t = t0; t < t1; ++t)
+      for (int c = ((blockIdx.y - e.ny) * NT + threadIdx.x) * 8; c < e.side_n;
+           c += (gridDim.y - e.ny) * NT * 8) {
+        float z[8];
+        load8(e.side_in + (int64_t)t * e.side_ld_in + c, z);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+          const float r = fmaxf(z[i], 0.f);
+          z[i] = r * r;
+        }
+        store8(e.side_out + (int64_t)t * e.side_ld_out + c, z);
+      }
+    return;
+  }
   const int l = threadIdx.x % LG, grp = threadIdx.x / LG;
-  const T* p = proj + (int64_t)t * ld_proj;
+  const int dim = a.dim, vdim = a.vdim, H = a.H, G = a.G, rot_dims = a.rot_dims;
   const int nq = H * dim, nk = G * dim, nv = G * vdim;
   const int half = rot_dims >> 1;
-  const float* cs = cosT + (int64_t)tok_pos[t] * half;
-  const float* sn = sinT + (int64_t)tok_pos[t] * half;
-  T* row = own_kv ? pool + (int64_t)tok_row[t] * (nk + nv) : nullptr;
-  const int jobs = own_kv ? H + 2 * G : H;
+  const int jobs = a.own_kv ? (a.v_from_k ? H + G : H + 2 * G) : H;
   const int c0 = l * 8;
-  // every lane of a wave walks the same number of rounds: the group sums
-  // below use whole-wave shuffles
-  for (int j0 = 0; j0 < jobs; j0 += NT / LG) {
+  // every lane of a wave walks the same number of rounds: the group sums and
+  // exchanges below use whole-wave shuffles
+  for (int j0 = blockIdx.y * (NT / LG); j0 < jobs; j0 += e.ny * (NT / LG)) {
     const int job = j0 + grp;
     const bool have = job < jobs;
     const bool is_v = have && job >= H + G;
     const bool is_q = have && job < H;
     const int n = is_v ? vdim : dim;
-    const T* in = p;
-    T* out = q_out;
-    if (is_q) {
-      in = p + job * dim;
-      out = q_out + (int64_t)t * nq + job * dim;
-    } else if (have && !is_v) {
-      in = p + nq + (job - H) * dim;
-      out = row + (job - H) * dim;
-    } else if (is_v) {
-      in = p + nq + nk + (job - H - G) * vdim;
-      out = row + nk + (job - H - G) * vdim;
-    }
     const bool act = have && c0 < n;
-    float x[8];
+    // first projected channel of this head, and of this lane
+    const int col = is_v ? nq + nk + (job - H - G) * vdim : (have ? job : 0) * dim;
+    const int ch = col + (act ? c0 : 0);
+    const bool turn = act && !is_v && c0 < rot_dims;
+    const bool second = turn && a.half && c0 >= half;
+    const int pc = !turn || !a.half ? c0 : (second ? c0 - half : c0 + half);
+    float wv[8], wc[TAPS > 0 ? 8 * TAPS : 1], hist[TAIL][8];
+    if (a.norm == 2 && act && !is_v) load8((is_q ? a.wq : a.wk) + c0, wv);
+    if (TAPS > 0) {
 #pragma unroll
-    for (int e = 0; e < 8; ++e) x[e] = 0.f;
-    if (act) load8(in + c0, x);
-    float ss = 0.f;
+      for (int i = 0; i < TAPS; ++i) {
+        float tmp[8];
+        load8(e.conv_w + (int64_t)ch * TAPS + 8 * i, tmp);
 #pragma unroll
-    for (int e = 0; e < 8; ++e) ss += x[e] * x[e];
-#pragma unroll
-    for (int o = 1; o < LG; o <<= 1) ss += __shfl_xor(ss, o, 64);
-    if (!act) continue;
-    if (is_v) {
-      if (v_eps >= 0.f) {
-        const float inv = rsqrtf(ss / (float)vdim + v_eps);
-#pragma unroll
-        for (int e = 0; e < 8; ++e) x[e] *= inv;
+        for (int u = 0; u < 8; ++u) wc[8 * i + u] = tmp[u];
       }
-      store8(out + c0, x);
-      continue;
     }
-    const float* w = is_q ? wq : wk;
-    const float inv = norm == 2 ? rsqrtf(ss / (float)dim + eps) : 1.f;
-    if (norm == 2) {
-      float wv[8];
-      load8(w + c0, wv);
+    for (int t = t0; t < t1; ++t) {
+      const int pos = a.tok_pos[t];
+      const T* p = proj + (int64_t)t * a.ld_proj;
+      float x[8];
 #pragma unroll
-      for (int e = 0; e < 8; ++e) x[e] *= inv * wv[e];
-    }
-    if (c0 < rot_dims) {
-      if (HALF) {  // the partner group sits half the rotated width away
-        const bool second = c0 >= half;
-        const int pc = second ? c0 - half : c0 + half;
-        const int f0 = second ? c0 - half : c0;
-        float o[8];
-        load8(in + pc, o);
-        if (norm == 2) {
-          float wv[8];
-          load8(w + pc, wv);
+      for (int i = 0; i < 8; ++i) x[i] = 0.f;
+      if (act) load8(p + ch, x);
+      if (TAPS > 0) {
+        const int s = e.tok_seq[t], j = t - e.cu[s];
+        if (TAPS > 1) {
+          T* sl = e.tails + (int64_t)e.seq_slot[s] * e.tail_stride + ch;
+          const int C = nq + nk + nv;
+          if (t == t0 || j == 0) {  // block-uniform: (re)load the earlier inputs
 #pragma unroll
-          for (int e = 0; e < 8; ++e) o[e] *= inv * wv[e];
+            for (int k = 1; k < TAPS; ++k) {
+#pragma unroll
+              for (int i = 0; i < 8; ++i) hist[k - 1][i] = 0.f;
+              if (pos - k >= 0 && act) {
+                if (k <= j)
+                  load8(p - (int64_t)k * a.ld_proj + ch, hist[k - 1]);
+                else
+                  load8(sl + (int64_t)(TAPS - 1 + j - k) * C, hist[k - 1]);
+              }
+            }
+          }
+          if (e.shift_tail && act) {  // oldest first: x(t-TAPS+2) .. x(t)
+#pragma unroll
+            for (int k = TAPS - 2; k >= 1; --k)
+              store8(sl + (int64_t)(TAPS - 2 - k) * C, hist[k - 1]);
+            store8(sl + (int64_t)(TAPS - 2) * C, x);
+          }
         }
+        float y[8];
 #pragma unroll
-        for (int e = 0; e < 8; ++e) {
-          const float co = cs[f0 + e], si = sn[f0 + e];
-          x[e] = second ? x[e] * co + o[e] * si : x[e] * co - o[e] * si;
+        for (int i = 0; i < 8; ++i) y[i] = wc[i * TAPS + TAPS - 1] * x[i];
+#pragma unroll
+        for (int k = 1; k < TAPS; ++k)
+#pragma unroll
+          for (int i = 0; i < 8; ++i) y[i] += wc[i * TAPS + TAPS - 1 - k] * hist[k - 1][i];
+#pragma unroll
+        for (int k = TAPS - 1; k >= 1; --k)
+#pragma unroll
+          for (int i = 0; i < 8; ++i) hist[k - 1][i] = k > 1 ? hist[k >= 2 ? k - 2 : 0][i] : x[i];
+#pragma unroll
+        for (int i = 0; i < 8; ++i) x[i] = act ? y[i] : 0.f;
+      }
+      T* row = a.own_kv ? pool + (int64_t)a.tok_row[t] * (nk + nv) : nullptr;
+      if (a.v_from_k && act && !is_q) store8(row + nk + (job - H) * dim + c0, x);
+      // norm in front of the rotation (or of a value head)
+      if (a.norm == 2 || a.v_eps >= 0.f) {
+        float ss = 0.f;
+#pragma unroll
+        for (int i = 0; i < 8; ++i) ss += x[i] * x[i];
+#pragma unroll
+        for (int o = 1; o < LG; o <<= 1) ss += __shfl_xor(ss, o, 64);
+        if (is_v) {
+          if (a.v_eps >= 0.f) {
+            const float inv = rsqrtf(ss / (float)vdim + a.v_eps);
+#pragma unroll
+            for (int i = 0; i < 8; ++i) x[i] *= inv;
+          }
+        } else if (a.norm == 2 && act) {
+          const float inv = rsqrtf(ss / (float)dim + a.eps);
+#pragma unroll
+          for (int i = 0; i < 8; ++i) x[i] *= inv * wv[i];
         }
-      } else {
+      }
+      if (rot_dims > 0) {
+        const float* cs = a.cosT + (int64_t)pos * half;
+        const float* sn = a.sinT + (int64_t)pos * half;
+        if (a.half) {  // the partner group sits half the rotated width away
+          const int src = (int)(threadIdx.x & 63) - l + (pc >> 3);
+          float o[8];
 #pragma unroll
-        for (int e = 0; e < 8; e += 2) {
-          if (c0 + e < rot_dims) {
-            const float co = cs[(c0 + e) >> 1], si = sn[(c0 + e) >> 1];
-            const float a = x[e], b = x[e + 1];
-            x[e] = a * co - b * si;
-            x[e + 1] = b * co + a * si;
+          for (int i = 0; i < 8; ++i) o[i] = __shfl(x[i], src, 64);
+          if (turn) {
+            const int f0 = second ? c0 - half : c0;
+            float co[8], si[8];
+            load8(cs + f0, co);
+            load8(sn + f0, si);
+#pragma unroll
+            for (int i = 0; i < 8; ++i)
+              x[i] = second ? x[i] * co[i] + o[i] * si[i] : x[i] * co[i] - o[i] * si[i];
+          }
+        } else if (turn) {
+#pragma unroll
+          for (int i = 0; i < 8; i += 2) {
+            if (c0 + i < rot_dims) {
+              const float co = cs[(c0 + i) >> 1], si = sn[(c0 + i) >> 1];
+              const float u = x[i], v = x[i + 1];
+              x[i] = u * co - v * si;
+              x[i + 1] = v * co + u * si;
+            }
           }
         }
       }
+      float f = is_q && a.qfac ? a.qfac[pos] : 1.f;
+      if (a.norm == 3) {
+        float ss = 0.f;
+#pragma unroll
+        for (int i = 0; i < 8; ++i) ss += x[i] * x[i];
+#pragma unroll
+        for (int o = 1; o < LG; o <<= 1) ss += __shfl_xor(ss, o, 64);
+        if (!is_v) f *= rsqrtf(ss / (float)dim + a.eps);
+      }
+      if (!act) continue;
+#pragma unroll
+      for (int i = 0; i < 8; ++i) x[i] *= f;
+      store8(is_q ? q_out + (int64_t)t * nq + job * dim + c0
+                  : (is_v ? row + nk + (job - H - G) * vdim : row + (job - H) * dim) + c0,
+             x);
     }
-    store8(out + c0, x);
   }
 }
 
@@ -1875,9 +2004,10 @@ int dsv_window_attn(const void* q, const void* pool, const int* tok_seq, const i
                     const int* table, int maxb, int bs, void* out, int ld_out, float* part,
                     int dt, int Ttok, int H, int G, int dim, int vdim, int KC, int nsplit,
                     float scale, int window, int keep_first, int chunk, float softcap,
-                    float out_scale, hipStream_t s) {
+                    float out_scale, const float* sink, const void* gate, int ld_gate,
+                    hipStream_t s) {
   if (vdim > WVPT * NT || H % G || nsplit < 1 || (nsplit > 1 && !part)) return -1;
-  if ((window > 0 && chunk > 0) || ld_out < H * vdim) return -3;
+  if ((window > 0 && chunk > 0) || ld_out < H * vdim || (gate && ld_gate < H)) return -3;
   if (Ttok <= 0) return 0;
   const int64_t lds = dsv_window_attn_lds(dt, dim, vdim, KC);
   if (lds > 64 * 1024) return -2;
@@ -1885,11 +2015,12 @@ int dsv_window_attn(const void* q, const void* pool, const int* tok_seq, const i
   BY_DTYPE(dt, (window_attn_k<T><<<grid, NT, lds, s>>>(
                    (const T*)q, (const T*)pool, tok_seq, tok_pos, table, maxb, bs, (T*)out, part,
                    ld_out, H, G, dim, vdim, KC, nsplit, scale, window, keep_first, chunk, softcap,
-                   nsplit > 1 ? 1.f : out_scale)));
+                   nsplit > 1 ? 1.f : out_scale, sink, (const T*)gate, ld_gate)));
   if (nsplit > 1) {
     dim3 g2(Ttok, H);
-    BY_DTYPE(dt, (window_attn_merge_k<T><<<g2, NT, 0, s>>>(part, (T*)out, ld_out, H, vdim,
-                                                           nsplit, out_scale)));
+    BY_DTYPE(dt, (window_attn_merge_k<T><<<g2, NT, 0, s>>>(
+                     part, (T*)out, ld_out, H, vdim, nsplit, out_scale, sink, (const T*)gate,
+                     ld_gate)));
   }
   return (int)hipGetLastError();
 }
@@ -1907,16 +2038,17 @@ int dsv_window_attn_mfma(const void* q, const void* pool, const int* work, int n
                          const int* cu, const int* seq_start, const int* table, int maxb, int bs,
                          void* out, int ld_out, float* part, int Ttok, int H, int G, int dim,
                          int vdim, int nsplit, float scale, int window, int keep_first,
-                         int chunk, float softcap, float out_scale, hipStream_t s) {
+                         int chunk, float softcap, float out_scale, const float* sink,
+                         const void* gate, int ld_gate, hipStream_t s) {
   if (!dsv_window_attn_mfma_ok(dim, vdim) || H % G) return -1;
-  if ((window > 0 && chunk > 0) || ld_out < H * vdim) return -4;
+  if ((window > 0 && chunk > 0) || ld_out < H * vdim || (gate && ld_gate < H)) return -4;
   if (nsplit < 1 || (nsplit > 1 && !part)) return -3;
   if (nwork <= 0) return 0;
 #define GO(DKT, DVB, PF)                                                                        \
   return launch_window_attn_mfma<DKT, DVB, PF>(q, pool, work, nwork, cu, seq_start, table, maxb, \
                                                bs, out, ld_out, part, Ttok, H, G, dim, vdim,     \
                                                nsplit, scale, window, keep_first, chunk,         \
-                                               softcap, out_scale, s)
+                                               softcap, out_scale, sink, gate, ld_gate, s)
   if (dim <= 64 && vdim <= 64) GO(4, 2, true);
   if (dim <= 128 && vdim <= 128) GO(8, 4, true);
   GO(16, 8, false);
@@ -2086,49 +2218,85 @@ int dsv_softplus_decay(const void* z, int ld_z, const float* bias, const float* 
   return (int)hipGetLastError();
 }
 
-// norm: 0 none, 2 per head (weights of size dim); half: rotary pairing
-// (i, i + rot_dims/2) instead of (2i, 2i+1); v_eps < 0: values pass unchanged.
+// 1 when the vector form of the per-head prologue covers these operands: whole
+// groups of 8 everywhere; with the half pairing a group's partner is a whole
+// group too. The convolution and the side activation exist in it only.
+int dsv_attn_prep_heads_vec(int ld_proj, int dim, int vdim, int rot_dims, int half, int taps) {
+  const int big = dim > vdim ? dim : vdim;
+  return dim % 8 == 0 && vdim % 8 == 0 && ld_proj % 8 == 0 && big <= 512 &&
+         (half ? rot_dims % 16 == 0 : 1) && taps >= 0 && taps <= 4 && taps != 1;
+}
+
+// norm: 0 none, 2 per head (weights of size dim), 3 per head after the
+// rotation, without weight; half: rotary pairing (i, i + rot_dims/2) instead
+// of (2i, 2i+1); v_eps < 0: values pass unchanged; v_from_k: values are the
+// projected keys. taps > 0: convolution first (vector form only); single: every
+// sequence of the step brings one token. side_n > 0: relu^2 of another slice.
 int dsv_attn_prep_heads(const void* proj, int ld_proj, const float* wq, const float* wk,
                         const int* tok_pos, const int* tok_row, const float* cosT,
-                        const float* sinT, void* pool, void* q_out, int dt, int Ttok, int H,
-                        int G, int dim, int vdim, int rot_dims, int own_kv, int norm, int half,
-                        float eps, float v_eps, hipStream_t s) {
+                        const float* sinT, const float* qfac, void* pool, void* q_out, int dt,
+                        int Ttok, int H, int G, int dim, int vdim, int rot_dims, int own_kv,
+                        int norm, int half, int v_from_k, float eps, float v_eps,
+                        const void* conv_w, void* tails, int64_t tail_stride, int taps,
+                        const int* cu, const int* seq_slot, const int* seq_start,
+                        const int* tok_seq, int nseq, int single, const void* side_in,
+                        int side_ld_in, void* side_out, int side_ld_out, int side_n,
+                        hipStream_t s) {
   if (rot_dims < 0 || (rot_dims & 1) || rot_dims > dim || H % G) return -1;
-  if ((norm != 0 && norm != 2) || (norm == 2 && (!wq || (own_kv && !wk)))) return -2;
+  if ((norm != 0 && norm != 2 && norm != 3) || (norm == 2 && (!wq || (own_kv && !wk)))) return -2;
   if (rot_dims > 0 && (!cosT || !sinT)) return -3;
+  if (v_from_k && (!own_kv || dim != vdim || taps > 0 || v_eps >= 0.f)) return -4;
+  const int C = H * dim + (own_kv ? G * dim + (v_from_k ? 0 : G * vdim) : 0);
+  if (ld_proj < C) return -5;
+  const bool vec = dsv_attn_prep_heads_vec(ld_proj, dim, vdim, rot_dims, half, taps) &&
+                   (uintptr_t)proj % 16 == 0;
+  const bool extra = taps > 0 || side_n > 0;
+  if (extra && !vec) return -6;
+  if (taps > 0 && (!own_kv || (taps > 1 && (!tails || tail_stride % 8)))) return -7;
+  if (side_n > 0 && (side_n % 8 || side_ld_in % 8 || side_ld_out % 8 ||
+                     (uintptr_t)side_in % 16 || (uintptr_t)side_out % 16))
+    return -8;
   if (Ttok <= 0) return 0;
-  const int big = dim > vdim ? dim : vdim;
-  // vector form: whole groups of 8 everywhere; with the half pairing a group's
-  // partner is a whole group too
-  const bool vec = dim % 8 == 0 && vdim % 8 == 0 && ld_proj % 8 == 0 && big <= 512 &&
-                   (half ? rot_dims % 16 == 0 : true) && (uintptr_t)proj % 16 == 0;
-#define PREPH(HALF, LG)                                                                        \
-  BY_DTYPE(dt, (attn_prep_heads_vec_k<T, HALF, LG><<<Ttok, NT, 0, s>>>(                         \
-                   (const T*)proj, ld_proj, wq, wk, tok_pos, tok_row, cosT, sinT, (T*)pool,    \
-                   (T*)q_out, H, G, dim, vdim, rot_dims, own_kv, norm, eps, v_eps)))
-#define PREPH_BY_LG(HALF)                        \
-  do {                                           \
-    if (big <= 32) PREPH(HALF, 4);               \
-    else if (big <= 64) PREPH(HALF, 8);          \
-    else if (big <= 128) PREPH(HALF, 16);        \
-    else if (big <= 256) PREPH(HALF, 32);        \
-    else PREPH(HALF, 64);                        \
-  } while (0)
-  if (vec) {
-    if (half) PREPH_BY_LG(true);
-    else PREPH_BY_LG(false);
+  PrepArgs a{ld_proj, H, G, dim, vdim, rot_dims, own_kv, norm, half, v_from_k, eps, v_eps,
+             wq, wk, cosT, sinT, qfac, tok_pos, tok_row};
+  if (!vec) {
+    BY_DTYPE(dt, (attn_prep_heads_k<T><<<Ttok, NT, 0, s>>>((const T*)proj, (T*)pool, (T*)q_out,
+                                                          a)));
     return (int)hipGetLastError();
   }
-#undef PREPH_BY_LG
-#undef PREPH
-  if (half)
-    BY_DTYPE(dt, (attn_prep_heads_k<T, true><<<Ttok, NT, 0, s>>>(
-                     (const T*)proj, ld_proj, wq, wk, tok_pos, tok_row, cosT, sinT, (T*)pool,
-                     (T*)q_out, H, G, dim, vdim, rot_dims, own_kv, norm, eps, v_eps)));
-  else
-    BY_DTYPE(dt, (attn_prep_heads_k<T, false><<<Ttok, NT, 0, s>>>(
-                     (const T*)proj, ld_proj, wq, wk, tok_pos, tok_row, cosT, sinT, (T*)pool,
-                     (T*)q_out, H, G, dim, vdim, rot_dims, own_kv, norm, eps, v_eps)));
+  const int big = dim > vdim ? dim : vdim;
+  const int jobs = own_kv ? (v_from_k ? H + G : H + 2 * G) : H;
+  const bool few = Ttok < 512;  // spread a token's heads over workgroups
+  const int toks = taps > 0 && !few ? 4 : 1;
+  const int blocks = (Ttok + toks - 1) / toks;
+#define PREPV(LG, TAPS)                                                                           \
+  do {                                                                                            \
+    const int ny = few ? (jobs + NT / LG - 1) / (NT / LG) : 1;                                    \
+    const int ns = side_n > 0 ? (few ? (side_n / 8 + NT - 1) / NT : 1) : 0;                       \
+    BY_DTYPE(dt, (attn_prep_heads_vec_k<T, LG, TAPS><<<dim3(blocks, ny + ns), NT, 0, s>>>(        \
+                     (const T*)proj, (T*)pool, (T*)q_out, Ttok, a,                                \
+                     PrepSteps<T>{(const T*)conv_w, (T*)tails, tail_stride, cu, seq_slot,         \
+                                  tok_seq, single, toks, ny, (const T*)side_in, (T*)side_out,     \
+                                  side_n, side_ld_in, side_ld_out})));                            \
+  } while (0)
+#define PREPV_BY_LG(TAPS)                  \
+  do {                                     \
+    if (big <= 32) PREPV(4, TAPS);         \
+    else if (big <= 64) PREPV(8, TAPS);    \
+    else if (big <= 128) PREPV(16, TAPS);  \
+    else if (big <= 256) PREPV(32, TAPS);  \
+    else PREPV(64, TAPS);                  \
+  } while (0)
+  if (taps == 4) PREPV_BY_LG(4);
+  else if (taps == 3) PREPV_BY_LG(3);
+  else if (taps == 2) PREPV_BY_LG(2);
+  else PREPV_BY_LG(0);
+#undef PREPV_BY_LG
+#undef PREPV
+  if (taps > 1 && !single)
+    BY_DTYPE(dt, (conv_tail_shift_k<T><<<nseq, NT, 0, s>>>((const T*)proj, ld_proj, (T*)tails,
+                                                           tail_stride, cu, seq_slot, seq_start,
+                                                           C, taps)));
   return (int)hipGetLastError();
 }
 

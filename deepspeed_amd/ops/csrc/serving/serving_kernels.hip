@@ -125,6 +125,81 @@ __global__ __launch_bounds__(NT) void layer_norm_vec_k(
   }
 }
 
+// --------------------------------------- residual add + dynamic tanh
+// x' = x + y and tanh(alpha * x') * w + b, elementwise (no statistic of the
+// row). Without idx the stream becomes x' in place (y null: it is only read);
+// with idx output row r reads rows idx[r] and leaves the stream alone. The
+// grid's stride is a whole number of rows, so a thread keeps its column (and
+// its weights) from row to row; VEC: eight columns per thread, two rows in
+// flight.
+// 16-bit results: 1 - 2 / (e^2z + 1), error of a few 1e-7
+__device__ __forceinline__ float tanh_fast(float z) {
+  const float e = __expf(2.f * z);
+  return 1.f - 2.f * __builtin_amdgcn_rcpf(e + 1.f);
+}
+template <typename TO> __device__ __forceinline__ float tanh_as(float z);
+template <> __device__ __forceinline__ float tanh_as<float>(float z) { return tanhf(z); }
+template <> __device__ __forceinline__ float tanh_as<bf16>(float z) { return tanh_fast(z); }
+
+template <typename TY, typename TO, bool VEC>
+__global__ __launch_bounds__(NT) void residual_tanh_k(
+    float* __restrict__ x, const TY* __restrict__ y, const float* __restrict__ alpha,
+    const float* __restrict__ w, const float* __restrict__ b, const int64_t* __restrict__ idx,
+    TO* __restrict__ h, int rows, int C) {
+  constexpr int V = VEC ? 8 : 1;
+  const int CV = C / V;
+  const int i0 = blockIdx.x * NT + threadIdx.x;
+  const int dr = gridDim.x * NT / CV;  // exact by the launch's choice of grid
+  const int c = (i0 % CV) * V;
+  const float al = alpha[0];
+  float wv[V], bv[V];
+  if constexpr (VEC) {
+    load8(w + c, wv);
+    load8(b + c, bv);
+  } else {
+    wv[0] = w[c];
+    bv[0] = b[c];
+  }
+  constexpr int U = 2;
+  for (int r0 = i0 / CV; r0 < rows; r0 += U * dr) {
+    float xv[U][V], yv[U][V];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int r = r0 + u * dr;
+      if (r < rows) {
+        const int64_t at = (idx ? idx[r] : (int64_t)r) * C + c;
+        if constexpr (VEC) {
+          load8(x + at, xv[u]);
+          if (y) load8(y + at, yv[u]);
+        } else {
+          xv[u][0] = x[at];
+          if (y) yv[u][0] = ld(y + at);
+        }
+      }
+    }
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int r = r0 + u * dr;
+      if (r < rows) {
+        const int64_t at = (int64_t)r * C + c;
+        float o[V];
+#pragma unroll
+        for (int i = 0; i < V; ++i) {
+          if (y) xv[u][i] += yv[u][i];
+          o[i] = tanh_as<TO>(al * xv[u][i]) * wv[i] + bv[i];
+        }
+        if constexpr (VEC) {
+          if (y && !idx) store8(x + at, xv[u]);
+          store8(h + at, o);
+        } else {
+          if (y && !idx) x[at] = xv[u][0];
+          st(h + at, o[0]);
+        }
+      }
+    }
+  }
+}
+
 // --------------------------------- residual add + layer norm + token shift
 // v = x[r] + mult * y[r] + extra (y, extra optional), h = layer norm of v with
 // weight and bias; x_out[r] (optional) = v. SHIFT: out[t] = h_t + (h_(t-1) -
@@ -1184,17 +1259,18 @@ __global__ __launch_bounds__(NT) void scaled_add_k(
 }
 
 // -------------------------------------------------- plain row activations
-// ACT: 0 = exact GELU (erf), 1 = tanh GELU, 2 = SiLU; z is a column slice
-// with row stride ld_z, out is contiguous.
+// ACT: 0 = exact GELU (erf), 1 = tanh GELU, 2 = SiLU, 3 = relu squared; z and
+// out are column slices with row strides ld_z and ld_out.
 template <int ACT>
 __device__ __forceinline__ float row_act(float z) {
   if (ACT == 0) return 0.5f * z * (1.f + erff(z * 0.70710678118654752f));
   if (ACT == 1) return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
+  if (ACT == 3) return z > 0.f ? z * z : 0.f;
   return z / (1.f + expf(-z));
 }
 
 template <typename T, int ACT, bool VEC>
-__global__ void act_rows_k(const T* __restrict__ z, int ld_z, T* __restrict__ out,
+__global__ void act_rows_k(const T* __restrict__ z, int ld_z, T* __restrict__ out, int ld_out,
                            int64_t rows, int F) {
   if (VEC) {
     const int F8 = F / 8;
@@ -1207,7 +1283,7 @@ __global__ void act_rows_k(const T* __restrict__ z, int ld_z, T* __restrict__ ou
       load8(z + r * ld_z + c, v);
 #pragma unroll
       for (int e = 0; e < 8; ++e) v[e] = row_act<ACT>(v[e]);
-      store8(out + r * F + c, v);
+      store8(out + r * ld_out + c, v);
     }
   } else {
     const int64_t n = rows * F;
@@ -1215,7 +1291,7 @@ __global__ void act_rows_k(const T* __restrict__ z, int ld_z, T* __restrict__ ou
          i += (int64_t)gridDim.x * blockDim.x) {
       const int64_t r = i / F;
       const int c = (int)(i - r * F);
-      st(out + i, row_act<ACT>(ld(z + r * ld_z + c)));
+      st(out + r * ld_out + c, row_act<ACT>(ld(z + r * ld_z + c)));
     }
   }
 }
@@ -1558,26 +1634,64 @@ int dsv_scaled_add(float* x, const float* s1, const void* y1, const float* s2, c
   return (int)hipGetLastError();
 }
 
-int dsv_act_rows(const void* z, int ld_z, void* out, int dt, int64_t rows, int F, int act,
-                 hipStream_t s) {
+int dsv_act_rows(const void* z, int ld_z, void* out, int ld_out, int dt, int64_t rows, int F,
+                 int act, hipStream_t s) {
   if (rows * F <= 0) return 0;
-  if (act < 0 || act > 2) return -1;
-  const bool vec = F % 8 == 0 && ld_z % 8 == 0 && (uintptr_t)z % 16 == 0;
+  if (act < 0 || act > 3 || ld_z < F || ld_out < F) return -1;
+  const bool vec = F % 8 == 0 && ld_z % 8 == 0 && ld_out % 8 == 0 && (uintptr_t)z % 16 == 0 &&
+                   (uintptr_t)out % 16 == 0;
   const int64_t n = vec ? rows * (F / 8) : rows * F;
   const int g = (int)((n + 255) / 256 > 262140 ? 262140 : (n + 255) / 256);
 #define AR(ACT)                                                                                 \
   do {                                                                                          \
     if (vec)                                                                                    \
       BY_DTYPE(dt, (act_rows_k<T, ACT, true><<<g, 256, 0, s>>>((const T*)z, ld_z, (T*)out,      \
-                                                               rows, F)));                      \
+                                                               ld_out, rows, F)));              \
     else                                                                                        \
       BY_DTYPE(dt, (act_rows_k<T, ACT, false><<<g, 256, 0, s>>>((const T*)z, ld_z, (T*)out,     \
-                                                                rows, F)));                     \
+                                                                ld_out, rows, F)));             \
   } while (0)
   if (act == 0) AR(0);
   else if (act == 1) AR(1);
-  else AR(2);
+  else if (act == 2) AR(2);
+  else AR(3);
 #undef AR
+  return (int)hipGetLastError();
+}
+
+// y may be null (y_dt is then ignored); idx null: all rows, x updated in place
+int dsv_residual_tanh(float* x, const void* y, int y_dt, const float* alpha, const float* w,
+                      const float* b, const int64_t* idx, void* h, int out_dt, int rows, int C,
+                      hipStream_t s) {
+  if (C < 1 || !x || !h) return -1;
+  if (rows <= 0) return 0;
+  const bool vec = C % 8 == 0;
+  const int cv = vec ? C / 8 : C;
+  if ((int64_t)rows * cv > (int64_t)1 << 30) return -2;
+  int m = cv, n = NT;  // whole rows per grid stride: blocks in multiples of cv / gcd(cv, NT)
+  while (n) {
+    const int r = m % n;
+    m = n;
+    n = r;
+  }
+  const int mult = cv / m;
+  const int per = rows >= 1024 ? 4 : 1;  // rows per thread
+  const int want = (int)(((int64_t)rows * cv + (int64_t)NT * per - 1) / ((int64_t)NT * per));
+  const int grid = (want + mult - 1) / mult * mult;
+#define RT(TY, TO, VEC)                                                                       \
+  residual_tanh_k<TY, TO, VEC><<<grid, NT, 0, s>>>(x, (const TY*)y, alpha, w, b, idx, (TO*)h, \
+                                                   rows, C)
+#define RT_BY(TY, TO)            \
+  do {                           \
+    if (vec) RT(TY, TO, true);   \
+    else RT(TY, TO, false);      \
+  } while (0)
+  if (y_dt == 0 && out_dt == 0) RT_BY(float, float);
+  else if (y_dt == 0) RT_BY(float, bf16);
+  else if (out_dt == 0) RT_BY(bf16, float);
+  else RT_BY(bf16, bf16);
+#undef RT_BY
+#undef RT
   return (int)hipGetLastError();
 }
 

@@ -334,3 +334,26 @@ def residual_norm(x, y, mult, weight, bias, eps, out_dtype=None, extra=None,
     if index is None and new is not x and shift is None:
         new = x.copy_(new)
     return (x if index is not None else new), h.to(out_dtype)
+
+
+def residual_tanh(x, y, alpha, weight, bias, out_dtype=None, index=None):
+    """Residual add on an fp32 stream and the dynamic tanh of the new rows in
+    one pass: ``x' = x + y``, ``h = tanh(alpha * x') * weight + bias`` (Zhu et
+    al., "Transformers without Normalization"). It takes no statistic of the
+    row, so it is elementwise. ``y`` ([T, C], any float type) may be None;
+    ``alpha`` is a one-element fp32 tensor, ``weight``/``bias`` are fp32 [C].
+    Without ``index`` x becomes x' in place; with it (int64 [R]) only those
+    rows are evaluated and the stream is left as it is. All fp32, rounded once
+    to ``out_dtype``. Returns h."""
+    assert x.dtype == torch.float32
+    out_dtype = out_dtype or torch.float32
+    if x.is_cuda and _sk().enabled():
+        return _sk().residual_tanh(x, y, alpha, weight, bias, out_dtype,
+                                   index)
+    new = x if index is None else x[index]
+    if y is not None:
+        new = new + (y if index is None else y[index]).float()
+        if index is None:
+            new = x.copy_(new)
+    return (torch.tanh(alpha.float().reshape(()) * new) * weight.float()
+            + bias.float()).to(out_dtype)

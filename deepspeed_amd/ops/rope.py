@@ -96,6 +96,21 @@ def rope_tables(dim: int, max_seq: int, theta: float = 500000.0,
     return _table_cache[key]
 
 
+_factor_cache = {}
+
+
+def temperature_table(max_seq: int, coef: float, every, device=None):
+    """fp32 [max_seq] factors on the queries of position p that grow with the
+    logarithm of the block p lies in: ``1 + coef * ln(floor((p + 1) / every)
+    + 1)`` (evaluated in fp64)."""
+    key = (max_seq, coef, every, str(device))
+    if key not in _factor_cache:
+        p = torch.arange(1, max_seq + 1, dtype=torch.float64)
+        _factor_cache[key] = (1.0 + coef * torch.log(
+            torch.floor(p / every) + 1.0)).float().to(device).contiguous()
+    return _factor_cache[key]
+
+
 def _torch_rope(x, cos, sin, positions=None, backward=False):
     B, S, H, D = x.shape
     half = D // 2

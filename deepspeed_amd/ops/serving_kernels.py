@@ -501,7 +501,8 @@ def _vp(t):
 
 def attn_prep(proj, batch, pool, q_norm_w, k_norm_w, eps, heads, kv_heads,
               dim, vdim, rot_dims, cos, sin, own_kv=True, norm="whole",
-              layout="interleaved", v_unit_eps=None):
+              layout="interleaved", v_unit_eps=None, conv=None,
+              v_from_k=False, q_factor=None, side=None):
     T = proj.shape[0]
     _rows_ok(proj)
     assert proj.dtype == pool.dtype and T == batch.n_tokens
@@ -510,8 +511,12 @@ def attn_prep(proj, batch, pool, q_norm_w, k_norm_w, eps, heads, kv_heads,
     if rot_dims:
         assert cos.shape[1] == rot_dims // 2 and cos.shape[0] >= batch.max_ctx
         assert cos.dtype == torch.float32 and sin.shape == cos.shape
+    plain = conv is None and not v_from_k and q_factor is None
     q = torch.empty(T, heads, dim, dtype=proj.dtype, device=proj.device)
-    if norm == "whole" and layout == "interleaved" and v_unit_eps is None:
+    if norm == "whole" and layout == "interleaved" and v_unit_eps is None \
+            and plain:
+        if side is not None:
+            act_rows(side[0], _ROW_ACTS.index(side[2]), side[1])
         assert proj.is_contiguous() and q_norm_w.numel() == heads * dim
         if own_kv:
             assert k_norm_w.numel() == kv_heads * dim
@@ -530,18 +535,60 @@ def attn_prep(proj, batch, pool, q_norm_w, k_norm_w, eps, heads, kv_heads,
     if norm == "head":
         assert q_norm_w.numel() == dim
         assert not own_kv or k_norm_w.numel() == dim
-    _check(_seq().dsv_attn_prep_heads(
+    lib, half = _seq(), 1 if layout == "half" else 0
+    taps = 0
+    if conv is not None:
+        conv_w, tails = conv
+        C, taps = conv_w.shape
+        assert conv_w.dtype == tails.dtype == proj.dtype
+        assert conv_w.is_contiguous() and C == proj.shape[1] and own_kv
+        assert tails.shape[1:] == (taps - 1, C)
+        assert tails.stride(2) == 1 and (taps == 1 or tails.stride(1) == C)
+    if q_factor is not None:
+        assert q_factor.dtype == torch.float32 and q_factor.dim() == 1
+        assert q_factor.numel() >= batch.max_ctx
+    vec = proj.data_ptr() % 16 == 0 and lib.dsv_attn_prep_heads_vec(
+        _i(proj.stride(0)), _i(dim), _i(vdim), _i(rot_dims), _i(half),
+        _i(taps)) == 1
+    if taps and not vec:        # sizes the fused form does not cover
+        proj = conv_silu_ragged(proj, conv_w, tails, batch, None, proj.dtype,
+                                None)
+        taps = 0
+    if side is not None:
+        z, z_out, act = side
+        if not (vec and act == "relu2" and _slice8(z) and _slice8(z_out)):
+            act_rows(z, _ROW_ACTS.index(act), z_out)
+            side = None
+        else:
+            assert z.shape == z_out.shape and z.shape[0] == T
+            assert z.dtype == z_out.dtype == proj.dtype
+    _check(lib.dsv_attn_prep_heads(
         _vp(proj), _i(proj.stride(0)),
         _p(_f32(q_norm_w) if norm == "head" else None),
         _p(_f32(k_norm_w) if norm == "head" and own_kv else None),
         _p(batch.tok_pos), _p(batch.tok_row), _p(cos if rot_dims else None),
-        _p(sin if rot_dims else None), _p(pool), _p(q), _i(_dt(proj)), _i(T),
-        _i(heads), _i(kv_heads), _i(dim), _i(vdim), _i(rot_dims),
-        _i(1 if own_kv else 0), _i(2 if norm == "head" else 0),
-        _i(1 if layout == "half" else 0), _f(eps),
-        _f(-1.0 if v_unit_eps is None else v_unit_eps), _stream()),
-        "attn_prep_heads")
+        _p(sin if rot_dims else None), _p(q_factor), _p(pool), _p(q),
+        _i(_dt(proj)), _i(T), _i(heads), _i(kv_heads), _i(dim), _i(vdim),
+        _i(rot_dims), _i(1 if own_kv else 0),
+        _i({None: 0, "head": 2, "after": 3}[norm]), _i(half),
+        _i(1 if v_from_k else 0), _f(eps),
+        _f(-1.0 if v_unit_eps is None else v_unit_eps),
+        _p(conv_w if taps else None), _vp(tails) if taps else _p(None),
+        _l(tails.stride(0) if taps else 0), _i(taps), _p(batch.cu),
+        _p(batch.seq_slot), _p(batch.seq_start), _p(batch.tok_seq),
+        _i(batch.n_seqs), _i(1 if single_tokens(batch) else 0),
+        _p(None) if side is None else _vp(z),
+        _i(0 if side is None else z.stride(0)),
+        _p(None) if side is None else _vp(z_out),
+        _i(0 if side is None else z_out.stride(0)),
+        _i(0 if side is None else z.shape[1]), _stream()), "attn_prep_heads")
     return q
+
+
+def _slice8(t):
+    """A 2-d operand of whole, aligned groups of eight values."""
+    return t.stride(1) == 1 and t.shape[1] % 8 == 0 and t.stride(0) % 8 == 0 \
+        and t.data_ptr() % 16 == 0
 
 
 def _window_tile_work(batch, kv_heads, rep, tile_rows, device):
@@ -570,7 +617,7 @@ def _window_tile_work(batch, kv_heads, rep, tile_rows, device):
 
 def window_attention(q, pool, batch, kv_heads, dim, vdim, scale, window=0,
                      keep_first=0, path=None, chunk=0, softcap=0.0,
-                     out_scale=1.0, out=None):
+                     out_scale=1.0, out=None, sink=None, gate=None):
     """``path`` forces "mfma" or "exact" (tests); default: the tile kernel for
     bf16 at head sizes it covers (prompt portions and, with split keys, single
     tokens), the exact kernel otherwise (fp32)."""
@@ -592,6 +639,14 @@ def window_attention(q, pool, batch, kv_heads, dim, vdim, scale, window=0,
     assert out.shape == (T, H * vdim) and out.stride(1) == 1
     assert out.dtype == q.dtype and out.is_cuda
     ld_out = out.stride(0)
+    if sink is not None:
+        assert sink.numel() == H
+        sink = _f32(sink).contiguous()
+    if gate is not None:
+        assert gate.shape == (T, H) and gate.dtype == q.dtype
+        _rows_ok(gate)
+    extra = (_p(sink), _p(None) if gate is None else _vp(gate),
+             _i(0 if gate is None else gate.stride(0)))
     mfma = q.dtype == torch.bfloat16 and \
         lib.dsv_window_attn_mfma_ok(_i(dim), _i(vdim)) == 1
     if path is None:
@@ -616,7 +671,7 @@ def window_attention(q, pool, batch, kv_heads, dim, vdim, scale, window=0,
             _i(batch.block_table.shape[1]), _i(batch.block_size), _vp(out),
             _i(ld_out), _p(part), _i(T), _i(H), _i(kv_heads), _i(dim),
             _i(vdim), _i(nsplit), _f(scale), _i(window), _i(keep_first),
-            _i(chunk), _f(softcap), _f(out_scale), _stream()),
+            _i(chunk), _f(softcap), _f(out_scale), *extra, _stream()),
             "window_attention(mfma)")
         return out
     kc = 64
@@ -638,7 +693,7 @@ def window_attention(q, pool, batch, kv_heads, dim, vdim, scale, window=0,
         _i(batch.block_size), _vp(out), _i(ld_out), _p(part), _i(dt), _i(T),
         _i(H), _i(kv_heads), _i(dim), _i(vdim), _i(kc), _i(nsplit), _f(scale),
         _i(window), _i(keep_first), _i(chunk), _f(softcap), _f(out_scale),
-        _stream()), "window_attention")
+        *extra, _stream()), "window_attention")
     return out
 
 
@@ -967,12 +1022,19 @@ def gated_add(x, g1, y1, g2, y2, norm_weight, eps, out_dtype, one_plus):
     return h
 
 
-def act_rows(z, act):
+_ROW_ACTS = ("gelu_erf", "gelu_tanh", "silu", "relu2")    # kernel's order
+
+
+def act_rows(z, act, out=None):
     T, F = z.shape
     _rows_ok(z)
-    out = torch.empty(T, F, dtype=z.dtype, device=z.device)
-    _check(load().dsv_act_rows(_vp(z), _i(z.stride(0)), _p(out), _i(_dt(z)),
-                               _l(T), _i(F), _i(act), _stream()), "act_rows")
+    if out is None:
+        out = torch.empty(T, F, dtype=z.dtype, device=z.device)
+    _rows_ok(out)
+    assert out.shape == z.shape and out.dtype == z.dtype
+    _check(load().dsv_act_rows(_vp(z), _i(z.stride(0)), _vp(out),
+                               _i(out.stride(0)), _i(_dt(z)), _l(T), _i(F),
+                               _i(act), _stream()), "act_rows")
     return out
 
 
@@ -1019,6 +1081,26 @@ def residual_norm(x, y, mult, weight, bias, eps, out_dtype, extra, shift,
         _p(h), _i(_DT[out_dtype]), _i(rows), _i(C), _f(eps), _stream()),
         "residual_norm")
     return new, h
+
+
+def residual_tanh(x, y, alpha, weight, bias, out_dtype, index):
+    T, C = x.shape
+    assert x.dtype == torch.float32 and x.is_contiguous()
+    assert alpha.numel() == 1 and weight.numel() == bias.numel() == C
+    if y is not None:
+        assert y.shape == x.shape
+        y = y.contiguous()
+    rows = T
+    if index is not None:
+        index = index.to(torch.int64).contiguous()
+        rows = index.numel()
+    h = torch.empty(rows, C, dtype=out_dtype, device=x.device)
+    _check(load().dsv_residual_tanh(
+        _p(x), _p(y), _i(0 if y is None else _dt(y)), _p(_f32(alpha)),
+        _p(_f32(weight).contiguous()), _p(_f32(bias).contiguous()), _p(index),
+        _p(h), _i(_DT[out_dtype]), _i(rows), _i(C), _stream()),
+        "residual_tanh")
+    return h
 
 
 # ------------------------------------------------ gated diagonal recurrence

@@ -34,7 +34,7 @@ def parse_args():
                    help="ZeRO-Offload optimizer states to host DRAM")
     p.add_argument("--activation-checkpointing", action="store_true")
     p.add_argument("--local_rank", type=int, default=-1)
-    p.add_argument("--serving", type=str, default=None, choices=["fizesun", "lolulorn", "savovik", "numolorn", "redudra"],
+    p.add_argument("--serving", type=str, default=None, choices=["fizesun", "lolulorn", "savovik", "numolorn", "redudra", "fubolix"],
                    help="instead of the training step: serving throughput "
                         "(prefill, decode) of this design beside Llama at "
                         "equal size, with per-kernel roofline distances")
@@ -46,8 +46,8 @@ def parse_args():
 
 def build_model(name, world_size=1):
     """Construct the model directly on the GPU in bf16 (random init on
-    device): building 8B on host fp32 took ~3 min of the round-1 bench
-    lease; on-device construction is seconds."""
+    device): building 8B on host fp32 took about 3
+    minutes; on-device construction is seconds."""
     torch.manual_seed(42)
     dev = torch.device("cuda") if torch.cuda.is_available() else         torch.device("cpu")
     if name.startswith("mixtral"):

@@ -248,12 +248,15 @@ class ContinuousBatcher:
         every token). This is the step the scheduler itself runs."""
         slots = [r.slot for r, _ in entries]
         counts = [len(t) for _, t in entries]
-        ids = torch.tensor([int(x) for _, t in entries for x in t],
-                           dtype=torch.long).to(self.device)
+        ids = [int(x) for _, t in entries for x in t]
+        n = len(ids)
+        if rows is not None:     # one transfer brings both
+            ids += [int(r) for r in rows]
+        ids = torch.tensor(ids, dtype=torch.long).to(self.device)
         self.cache.begin_ragged(slots, counts)
         try:
             if rows is not None:
-                rows = torch.as_tensor(rows, dtype=torch.long).to(self.device)
+                ids, rows = ids[:n], ids[n:]
             logits = self.model(ids, kv_cache=self.cache, rows=rows)
         finally:
             self.cache.end_step()

@@ -29,6 +29,11 @@ attention beside retention, alternating, dense feed-forwards) beside Savovik
 (its closest sibling: parallel attention and recurrence on the ragged path),
 Lolulorn and Llama; every kernel on its path is timed next to the like kernel
 of those paths.
+
+``--serving fubolix`` runs Fubolix (windowed attention whose values are its
+keys / convolved attention / windowed / causal attention with query temperature,
+parallel dense feed-forwards) beside Savovik (its closest sibling: parallel
+layers over the same attention module), Lolulorn and Llama.
 """
 
 import json
@@ -1374,6 +1379,197 @@ def run_redudra(sizes=("s", "m", "l"), kernels=True):
     return report
 
 
+# -------------------------------------------------------------- Fubolix
+def fubolix_config(z, vocab=32000):
+    """[windowed attention on its own keys, convolved attention, windowed
+    attention, causal attention with query temperature] repeated to
+    ``layers``; heads of 128, 4 query heads per key/value head, window 1024 + 4
+    kept tokens; dense feed-forwards beside every mixer."""
+    H = z["heads"]
+    att = {"heads": H, "kv_heads": max(1, H // 4), "dim": 128, "vdim": 128,
+           "scale": 128 ** -0.5}
+    yarn = {"factor": 2.0, "original": 2048, "fast": 32.0, "slow": 1.0}
+    mix = {"attention": {**att, "mask": {"size": 1024, "keep_first": 4},
+                         "rot": {"base": 500000.0, "dims": 64,
+                                 "scaling": yarn}},
+           "attention_2": {**att, "q_temp": {"coef": 0.1, "every": 1024}},
+           "attention_3": {**att, "conv": 4,
+                           "rot": {"base": 10000.0, "dims": 128,
+                                   "scaling": yarn}}}
+    order = ("attention", "attention_3", "attention", "attention_2")
+    layers = [{"type": order[i % 4], "mixer": mix[order[i % 4]],
+               "mlp": {"kind": "dense", "ff": z["ff"]}}
+              for i in range(z["layers"])]
+    return {"architecture": "Fubolix", "vocab": vocab, "width": z["width"],
+            "norm": {"eps": 1e-6}, "embedding": {"scale": 1.0},
+            "layers": layers}
+
+
+@torch.no_grad()
+def _fubolix_kernel_rows(z, dev):
+    """Every kernel on Fubolix's path at this size, each followed by the like
+    kernel of the Lolulorn or Savovik path at the same shapes ("like" names
+    it; rows with an empty "like" are the siblings themselves)."""
+    from ..ops import serving_kernels as sk
+    from ..ops.activations import act_rows
+    from ..ops.causal_conv import conv_silu_ragged
+    from ..ops.norms import residual_tanh
+    from ..ops.rope import rope_tables, temperature_table
+    from ..ops.window_attention import attn_prep
+    from .state_cache import PagedStateCache
+    bf = torch.bfloat16
+    B, S, W, H, F = z["batch"], z["seq"], z["width"], z["heads"], z["ff"]
+    G, d, dv, taps = max(1, H // 4), 128, 128, 4
+    C = H * d + G * (d + dv)
+    out = []
+
+    def row(name, like, fn, nbytes, flops=0.0, iters=5):
+        t = min(_timed(fn, 2, iters), _timed(fn, 1, iters))
+        bound = max(nbytes / HBM_BW, flops / MFMA_BF16)
+        out.append({"kernel": name, "like": like, "us": 1e6 * t,
+                    "bound_us": 1e6 * bound, "distance": t / bound})
+
+    al, wn, bn = (torch.full((n,), v, device=dev)
+                  for n, v in ((1, 0.5), (W, 1.0), (W, 0.0)))
+    qw, kw = torch.ones(H * d, device=dev), torch.ones(G * d, device=dev)
+    hw = torch.ones(d, device=dev)
+    cw = (torch.randn(C, taps, device=dev) * 0.4).to(bf)
+    for NB, n in ((B, S), (B, 1), (64, 1)):
+        T, held = NB * n, 0 if n > 1 else S
+        case = ", %d x %d tokens" % (NB, n)
+        cache = PagedStateCache([G * (d + dv)], {"conv": (taps - 1, C)}, NB,
+                                NB * (S + 64), dtype=bf, device=dev)
+        for i in range(NB):
+            cache.lens[i] = held
+        batch = cache.begin_ragged(list(range(NB)), [n] * NB)
+        pool, tails = cache.pools[0], cache.states["conv"]
+        # ---- residual add + dynamic tanh against the post-norm residual
+        x32 = torch.randn(T, W, device=dev)
+        y1 = (torch.randn(T, W, device=dev) * 0.01).to(bf)
+        row("residual_tanh (fp32 stream += bf16, bf16 out)" + case,
+            "layer_norm_add",
+            lambda: residual_tanh(x32, y1, al, wn, bn, bf), T * W * 12)
+        row("layer_norm_add (lolulorn)" + case, "",
+            lambda: sk.layer_norm_add(x32, y1, wn, bn, 1e-6, bf), T * W * 12)
+        # ---- prologues, alone and with the activation they carry along
+        cos, sin = rope_tables(d, cache.max_seq, 10000.0, device=dev)
+        c64, s64 = rope_tables(64, cache.max_seq, 10000.0, device=dev)
+        tab = temperature_table(cache.max_seq, 0.1, 1024, dev)
+        proj = torch.randn(T, C + F, device=dev).to(bf)
+        both = torch.empty(T, H * dv + F, device=dev, dtype=bf)
+        side = (proj[:, C:], both[:, H * dv:], "relu2")
+        act_bytes = T * F * 4
+        nk = (H + G) * d
+        plain = proj[:, :C].contiguous()
+        wide = T * C * 4
+
+        def after(side=None):
+            return attn_prep(proj[:, :nk], batch, pool, None, None, 1e-6, H,
+                             G, d, d, 64, c64, s64, norm="after",
+                             v_from_k=True, side=side)
+
+        def tempered(side=None):
+            return attn_prep(proj[:, :C], batch, pool, hw, hw, 1e-6, H, G, d,
+                             dv, 0, None, None, norm="head", q_factor=tab,
+                             side=side)
+
+        def convolved(side=None):
+            return attn_prep(proj[:, :C], batch, pool, None, None, 1e-6, H, G,
+                             d, dv, d, cos, sin, norm=None, layout="half",
+                             conv=(cw, tails), side=side)
+
+        def half_rotated(p):
+            return attn_prep(p, batch, pool, None, None, 1e-6, H, G, d, dv, d,
+                             cos, sin, norm=None, layout="half")
+
+        row("attn_prep: rotary, unit RMS after it, keys as values" + case,
+            "attn_prep (lolulorn", after, T * (nk + C) * 2)
+        row("attn_prep: per-head q/k norm, query temperature" + case,
+            "attn_prep (lolulorn", tempered, wide)
+        row("attn_prep (lolulorn: whole-projection norms, rotary)" + case, "",
+            lambda: sk.attn_prep(plain, batch, pool, qw, kw, 1e-6, H, G, d,
+                                 dv, d, cos, sin, True), wide)
+        row("attn_prep: convolution of %d taps, rotate-half" % taps + case,
+            "conv, then attn_prep", convolved, wide)
+        row("conv, then attn_prep (the two calls of redudra's parts)" + case,
+            "", lambda: half_rotated(conv_silu_ragged(
+                plain, cw, tails, batch, None, bf, None)), 2 * wide)
+        row("attn_prep with relu^2 beside it" + case,
+            "attn_prep, then act_rows", lambda: after(side),
+            T * (nk + C) * 2 + act_bytes)
+        row("attn_prep, then act_rows gelu_erf (savovik)" + case, "",
+            lambda: (half_rotated(plain), act_rows(proj[:, C:], "gelu_erf")),
+            wide + act_bytes)
+        if n > 1:       # ---- prefill attention: the kernel is the same one
+            q = after()
+            io = T * H * (d + dv) * 2 + T * G * (d + dv) * 2
+            gate = torch.randn(T, H, device=dev).to(bf)
+            sink = torch.zeros(H, device=dev)
+            win = 1024
+            seen = {0: S * (S + 1) // 2,
+                    win: sum(min(i + 1, win) + min(4, max(0, i + 1 - win))
+                             for i in range(S))}
+            for w, keep, g, tag in ((win, 4, gate, "window, sink and gate"),
+                                    (0, 0, None, "causal, sink")):
+                def att(s, gt, o):
+                    return sk.window_attention(
+                        q, pool, batch, G, d, dv, d ** -0.5, w, keep, out=o,
+                        sink=s, gate=gt)
+
+                fl = 2.0 * B * H * seen[w] * (d + dv)
+                name = tag.split(",")[0]
+                row("window_attention prefill: " + tag + case,
+                    "plain %s attention" % name,
+                    lambda: att(sink, g, both[:, :H * dv]), io, fl, iters=2)
+                row("plain %s attention (lolulorn)" % name + case, "",
+                    lambda: att(None, None, None), io, fl, iters=2)
+            del q
+        else:
+            pool.normal_()
+            q = (torch.randn(T, H, d, device=dev) * 0.1).to(bf)
+            gate = torch.randn(T, H, device=dev).to(bf)
+            sink = torch.zeros(H, device=dev)
+            for w, keep, g, tag in ((1024, 4, gate, "window, sink and gate"),
+                                    (0, 0, None, "causal, sink")):
+                def att(s, gt, o):
+                    return sk.window_attention(
+                        q, pool, batch, G, d, dv, d ** -0.5, w, keep, out=o,
+                        sink=s, gate=gt)
+
+                keys = min(S + 1, w + keep) if w else S + 1
+                nbytes = NB * keys * G * (d + dv) * 2
+                name = tag.split(",")[0]
+                row("window_attention decode: " + tag + case,
+                    "plain %s attention" % name,
+                    lambda: att(sink, g, both[:, :H * dv]), nbytes)
+                row("plain %s attention (lolulorn)" % name + case, "",
+                    lambda: att(None, None, None), nbytes)
+        cache.end_step()
+        del cache, pool, tails, proj, plain, both, side, x32, y1
+        torch.cuda.empty_cache()
+    return out
+
+
+def run_fubolix(sizes=("s", "m", "l"), kernels=True):
+    dev = torch.device("cuda", torch.cuda.current_device())
+    report = {}
+    for name in sizes:
+        z = dict(SIZES[name])
+        z["layers"] = 4
+        rec = {"size": {k: z[k] for k in z},
+               "fubolix": _ragged_throughput(fubolix_config(z), z, dev),
+               "savovik": _ragged_throughput(savovik_config(z), z, dev),
+               "lolulorn": _ragged_throughput(lolulorn_config(z), z, dev),
+               "llama": _llama_throughput(z, dev)}
+        if kernels:
+            rows = _fubolix_kernel_rows(z, dev)
+            rec["kernels"] = rows
+            rec["distance_over_sibling"] = _sibling_ratios(rows)
+        report[name] = rec
+        torch.cuda.empty_cache()
+    return report
+
+
 def _same_case(a, b):
     """Rows of one case carry the same '<n> requests' / '<n> x <m> tokens'."""
     import re
@@ -1397,55 +1593,23 @@ def run(sizes=("s", "m", "l"), kernels=True):
 
 def main(sizes="s,m,l", out=None, model="fizesun"):
     names = tuple(sizes.split(","))
-    if model == "redudra":
-        rep = run_redudra(names)
+    siblings = {"fubolix": (run_fubolix, ("savovik", "lolulorn", "llama")),
+                "redudra": (run_redudra, ("savovik", "lolulorn", "llama")),
+                "numolorn": (run_numolorn, ("lolulorn", "fizesun", "llama")),
+                "savovik": (run_savovik, ("lolulorn", "llama"))}
+    if model in siblings:
+        runner, others = siblings[model]
+        rep = runner(names)
         if out:
             with open(out, "w") as f:
                 json.dump(rep, f, indent=1)
         best = rep[names[-1]]
         print(json.dumps({
-            "metric": "redudra_serving_tokens_per_s", "unit": "tokens/s",
+            "metric": "%s_serving_tokens_per_s" % model, "unit": "tokens/s",
             "dtype": "bf16", "data": "synthetic", "n_gpus": 1,
-            "value": best["redudra"]["prefill_tok_s"],
+            "value": best[model]["prefill_tok_s"],
             "higher_is_better": True,
-            "sizes": {k: {"redudra": v["redudra"], "savovik": v["savovik"],
-                          "lolulorn": v["lolulorn"], "llama": v["llama"],
-                          "worst_distance_over_sibling": max(
-                              v.get("distance_over_sibling", {}).values(),
-                              default=None)}
-                      for k, v in rep.items()}}))
-        return rep
-    if model == "numolorn":
-        rep = run_numolorn(names)
-        if out:
-            with open(out, "w") as f:
-                json.dump(rep, f, indent=1)
-        best = rep[names[-1]]
-        print(json.dumps({
-            "metric": "numolorn_serving_tokens_per_s", "unit": "tokens/s",
-            "dtype": "bf16", "data": "synthetic", "n_gpus": 1,
-            "value": best["numolorn"]["prefill_tok_s"],
-            "higher_is_better": True,
-            "sizes": {k: {"numolorn": v["numolorn"], "lolulorn": v["lolulorn"],
-                          "fizesun": v["fizesun"], "llama": v["llama"],
-                          "worst_distance_over_sibling": max(
-                              v.get("distance_over_sibling", {}).values(),
-                              default=None)}
-                      for k, v in rep.items()}}))
-        return rep
-    if model == "savovik":
-        rep = run_savovik(names)
-        if out:
-            with open(out, "w") as f:
-                json.dump(rep, f, indent=1)
-        best = rep[names[-1]]
-        print(json.dumps({
-            "metric": "savovik_serving_tokens_per_s", "unit": "tokens/s",
-            "dtype": "bf16", "data": "synthetic", "n_gpus": 1,
-            "value": best["savovik"]["prefill_tok_s"],
-            "higher_is_better": True,
-            "sizes": {k: {"savovik": v["savovik"], "lolulorn": v["lolulorn"],
-                          "llama": v["llama"],
+            "sizes": {k: {**{m: v[m] for m in (model,) + others},
                           "worst_distance_over_sibling": max(
                               v.get("distance_over_sibling", {}).values(),
                               default=None)}

@@ -330,30 +330,37 @@ __global__ __launch_bounds__(NT) void window_attn_k(
   }
 }
 
+inline int merge_threads(int vdim) { return vdim <= 64 ? 64 : (vdim <= 128 ? 128 : NT); }
+
+// Every wave holds the splits' factors in its lanes (nsplit <= 64) and walks the
+// partial sums once.
 template <typename T>
 __global__ __launch_bounds__(NT) void window_attn_merge_k(
     const float* __restrict__ part, T* __restrict__ out, int ld_out, int H, int vdim,
     int nsplit, float out_scale, const float* __restrict__ sink, const T* __restrict__ gate,
     int ld_gate) {
-  const int t = blockIdx.x, h = blockIdx.y;
-  float m = -INFINITY;
-  for (int s = 0; s < nsplit; ++s) {
-    const float* pp = part + (((int64_t)t * nsplit + s) * H + h) * (vdim + 2);
-    if (pp[1] > 0.f) m = fmaxf(m, pp[0]);
+  const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x & 63;
+  const int64_t step = (int64_t)H * (vdim + 2);
+  const float* pp = part + ((int64_t)t * nsplit * H + h) * (vdim + 2);
+  float ms = -INFINITY, ls = 0.f;
+  if (lane < nsplit) {
+    ls = pp[lane * step + 1];
+    if (ls > 0.f) ms = pp[lane * step];
   }
-  float l = 0.f;
-  for (int s = 0; s < nsplit; ++s) {
-    const float* pp = part + (((int64_t)t * nsplit + s) * H + h) * (vdim + 2);
-    if (pp[1] > 0.f) l += pp[1] * expf(pp[0] - m);
-  }
+  const float m = wave_max(ms);
+  const float w = ls > 0.f ? expf(ms - m) : 0.f;
+  const float l = wave_sum(ls * w);
   const float f = head_factor(l, m, t, h, out_scale, sink, gate, ld_gate);
-  for (int c = threadIdx.x; c < vdim; c += NT) {
-    float a = 0.f;
+  for (int c = threadIdx.x; c < vdim; c += blockDim.x) {
+    float acc = 0.f;
+#pragma unroll 4
     for (int s = 0; s < nsplit; ++s) {
-      const float* pp = part + (((int64_t)t * nsplit + s) * H + h) * (vdim + 2);
-      if (pp[1] > 0.f) a += pp[2 + c] * expf(pp[0] - m);
+      const float ws = __uint_as_float(__builtin_amdgcn_readlane(__float_as_uint(w), s));
+      // a split that saw no key has written no sums
+      const float v = ws > 0.f ? pp[s * step + 2 + c] : 0.f;
+      acc += ws * v;
     }
-    st(out + (int64_t)t * ld_out + h * vdim + c, a * f);
+    st(out + (int64_t)t * ld_out + h * vdim + c, acc * f);
   }
 }
 
@@ -712,7 +719,7 @@ int launch_window_attn_mfma(const void* q, const void* pool, const int* work, in
                                              keep_first, chunk, softcap, out_scale, sink,
                                              (const bf16*)gate, ld_gate);
   if (nsplit > 1)
-    window_attn_merge_k<bf16><<<dim3(Ttok, H), NT, 0, s>>>(
+    window_attn_merge_k<bf16><<<dim3(Ttok, H), merge_threads(vdim), 0, s>>>(
         part, (bf16*)out, ld_out, H, vdim, nsplit, out_scale, sink, (const bf16*)gate, ld_gate);
   return (int)hipGetLastError();
 }
@@ -855,7 +862,7 @@ __global__ __launch_bounds__(NT) void delta_prep_vec_k(
   }
 }
 
-// One block per sequence: the tail becomes the sequence's last taps-1 inputs
+// Workgroups (sequence, channels): the tail becomes the sequence's last taps-1 inputs
 // (from this step's rows, or shifted out of the old tail for short steps).
 template <typename T>
 __global__ __launch_bounds__(NT) void conv_tail_shift_k(
@@ -867,7 +874,7 @@ __global__ __launch_bounds__(NT) void conv_tail_shift_k(
   const int start = seq_start[s];
   const int count = cu[s + 1] - cu[s];
   T* sl = state + (int64_t)seq_slot[s] * state_slot_stride;
-  for (int c = threadIdx.x; c < C; c += NT) {
+  for (int c = blockIdx.y * NT + threadIdx.x; c < C; c += gridDim.y * NT) {
     for (int i = 0; i < tail; ++i) {  // ascending: reads stay ahead of writes
       const int p = start + count - tail + i;  // position kept at i
       T v;
@@ -1647,23 +1654,64 @@ __global__ __launch_bounds__(NT) void ssd_prep_vec_k(
 }
 
 // The per-head prologue with eight values per lane: a head is shared by LG
-// lanes (a power of two, 8 * LG >= dim and vdim); all sizes multiples of 8.
-// Two more steps share the launch:
+// lanes (a power of two, 8 * LG >= dim and vdim); all sizes multiples of 8. The
+// units of work, `toks` neighbouring tokens of one head, are laid out flat over
+// groups of LG lanes, so neither a short step nor an odd number of heads leaves
+// lanes idle. Two more steps share the launch:
 // * TAPS > 0: a short causal convolution over every projected channel first
 //   (weights [channels, TAPS]; earlier inputs come from this step's rows, from
-//   the slot's tail, or are zero). A workgroup takes `toks` neighbouring tokens
-//   so that weights and earlier rows stay in registers from one token to the
-//   next. shift_tail: every sequence brings exactly one token, so the lane that
-//   reads a channel's tail is its only reader and moves it on in place.
-// * side: workgroups with blockIdx.y >= ny square the positive part of another
-//   column slice (the feed-forward's first product).
+//   the slot's tail, or are zero). A group takes up to PREP_TOKS tokens: rows
+//   are fetched two tokens ahead, weights and earlier rows stay in registers
+//   (packed as they are stored) from one token to the next. shift_tail: every
+//   sequence brings exactly one token, so the lane that reads a channel's tail
+//   is its only reader and moves it on in place.
+// * side: workgroups past n_prep square the positive part of another column
+//   slice (the feed-forward's first product).
+constexpr int PREP_TOKS = 8;
+
+// eight values as they are stored
+template <typename T> struct Raw8;
+template <> struct Raw8<float> {
+  float4 a, b;
+  __device__ __forceinline__ void keep_packed() {}
+  __device__ __forceinline__ void zero() { a = b = make_float4(0.f, 0.f, 0.f, 0.f); }
+  __device__ __forceinline__ void load(const float* p) {
+    a = *reinterpret_cast<const float4*>(p);
+    b = *reinterpret_cast<const float4*>(p + 4);
+  }
+  __device__ __forceinline__ void store(float* p) const {
+    *reinterpret_cast<float4*>(p) = a;
+    *reinterpret_cast<float4*>(p + 4) = b;
+  }
+  __device__ __forceinline__ void widen(float (&x)[8]) const {
+    x[0] = a.x; x[1] = a.y; x[2] = a.z; x[3] = a.w;
+    x[4] = b.x; x[5] = b.y; x[6] = b.z; x[7] = b.w;
+  }
+};
+template <> struct Raw8<bf16> {
+  uint4 w;
+  // keeps the widened values from being carried through a loop in place of w
+  __device__ __forceinline__ void keep_packed() {
+    asm volatile("" : "+v"(w.x), "+v"(w.y), "+v"(w.z), "+v"(w.w));
+  }
+  __device__ __forceinline__ void zero() { w = make_uint4(0, 0, 0, 0); }
+  __device__ __forceinline__ void load(const bf16* p) { w = *reinterpret_cast<const uint4*>(p); }
+  __device__ __forceinline__ void store(bf16* p) const { *reinterpret_cast<uint4*>(p) = w; }
+  __device__ __forceinline__ void widen(float (&x)[8]) const {
+    x[0] = __uint_as_float(w.x << 16); x[1] = __uint_as_float(w.x & 0xffff0000u);
+    x[2] = __uint_as_float(w.y << 16); x[3] = __uint_as_float(w.y & 0xffff0000u);
+    x[4] = __uint_as_float(w.z << 16); x[5] = __uint_as_float(w.z & 0xffff0000u);
+    x[6] = __uint_as_float(w.w << 16); x[7] = __uint_as_float(w.w & 0xffff0000u);
+  }
+};
+
 template <typename T>
 struct PrepSteps {
   const T* conv_w;
   T* tails;
   int64_t tail_stride;
   const int *cu, *seq_slot, *tok_seq;
-  int shift_tail, toks, ny;
+  int shift_tail, toks, n_prep;
   const T* side_in;
   T* side_out;
   int side_n, side_ld_in, side_ld_out;
@@ -1674,160 +1722,180 @@ __global__ __launch_bounds__(NT) void attn_prep_heads_vec_k(
     const T* __restrict__ proj, T* __restrict__ pool, T* __restrict__ q_out, int Ttok, PrepArgs a,
     PrepSteps<T> e) {
   constexpr int TAIL = TAPS > 1 ? TAPS - 1 : 1;
-  const int t0 = blockIdx.x * e.toks, t1 = min(Ttok, t0 + e.toks);
-  if ((int)blockIdx.y >= e.ny) {
-    for (int t = t0; t < t1; ++t)
-      for (int c = ((blockIdx.y - e.ny) * NT + threadIdx.x) * 8; c < e.side_n;
-           c += (gridDim.y - e.ny) * NT * 8) {
-        float z[8];
-        load8(e.side_in + (int64_t)t * e.side_ld_in + c, z);
+  if ((int)blockIdx.x >= e.n_prep) {
+    const int n8 = e.side_n >> 3;
+    const int i = ((int)blockIdx.x - e.n_prep) * NT + threadIdx.x;
+    const int t = i / n8, c = (i - t * n8) * 8;
+    if (t >= Ttok) return;
+    float z[8];
+    load8(e.side_in + (int64_t)t * e.side_ld_in + c, z);
 #pragma unroll
-        for (int i = 0; i < 8; ++i) {
-          const float r = fmaxf(z[i], 0.f);
-          z[i] = r * r;
-        }
-        store8(e.side_out + (int64_t)t * e.side_ld_out + c, z);
-      }
+    for (int u = 0; u < 8; ++u) {
+      const float r = fmaxf(z[u], 0.f);
+      z[u] = r * r;
+    }
+    store8(e.side_out + (int64_t)t * e.side_ld_out + c, z);
     return;
   }
-  const int l = threadIdx.x % LG, grp = threadIdx.x / LG;
   const int dim = a.dim, vdim = a.vdim, H = a.H, G = a.G, rot_dims = a.rot_dims;
   const int nq = H * dim, nk = G * dim, nv = G * vdim;
   const int half = rot_dims >> 1;
   const int jobs = a.own_kv ? (a.v_from_k ? H + G : H + 2 * G) : H;
+  const int l = threadIdx.x % LG;
+  const int unit = blockIdx.x * (NT / LG) + threadIdx.x / LG;
+  const int span = unit / jobs, job = unit - span * jobs;
+  const int t0 = span * e.toks;
   const int c0 = l * 8;
-  // every lane of a wave walks the same number of rounds: the group sums and
-  // exchanges below use whole-wave shuffles
-  for (int j0 = blockIdx.y * (NT / LG); j0 < jobs; j0 += e.ny * (NT / LG)) {
-    const int job = j0 + grp;
-    const bool have = job < jobs;
-    const bool is_v = have && job >= H + G;
-    const bool is_q = have && job < H;
-    const int n = is_v ? vdim : dim;
-    const bool act = have && c0 < n;
-    // first projected channel of this head, and of this lane
-    const int col = is_v ? nq + nk + (job - H - G) * vdim : (have ? job : 0) * dim;
-    const int ch = col + (act ? c0 : 0);
-    const bool turn = act && !is_v && c0 < rot_dims;
-    const bool second = turn && a.half && c0 >= half;
-    const int pc = !turn || !a.half ? c0 : (second ? c0 - half : c0 + half);
-    float wv[8], wc[TAPS > 0 ? 8 * TAPS : 1], hist[TAIL][8];
-    if (a.norm == 2 && act && !is_v) load8((is_q ? a.wq : a.wk) + c0, wv);
+  const bool is_v = job >= H + G, is_q = job < H;
+  // lanes without work stay: the sums and exchanges below are whole-wave
+  const bool lane_on = t0 < Ttok && c0 < (is_v ? vdim : dim);
+  // first projected channel of this head, and of this lane
+  const int col = is_v ? nq + nk + (job - H - G) * vdim : job * dim;
+  const int ch = col + (lane_on ? c0 : 0);
+  const bool turn = lane_on && !is_v && c0 < rot_dims;
+  const bool second = turn && a.half && c0 >= half;
+  const int pc = !turn || !a.half ? c0 : (second ? c0 - half : c0 + half);
+  float wv[8];
+  if (a.norm == 2 && lane_on && !is_v) load8((is_q ? a.wq : a.wk) + c0, wv);
+  Raw8<T> wc[TAPS > 0 ? TAPS : 1], hist[TAIL], next[2];
+  if (TAPS > 0) {
+#pragma unroll
+    for (int i = 0; i < TAPS; ++i) wc[i].load(e.conv_w + (int64_t)ch * TAPS + 8 * i);
+  }
+  auto fetch = [&](int k, Raw8<T>& r) {
+    r.zero();
+    if (lane_on && k < e.toks && t0 + k < Ttok) r.load(proj + (int64_t)(t0 + k) * a.ld_proj + ch);
+  };
+  fetch(0, next[0]);
+  if (TAPS > 0) fetch(1, next[1]);
+  int s = 0, j = 0, end = -1, pos = 0;  // sequence, place in the step, its end
+#pragma unroll 1
+  for (int k = 0; k < e.toks; ++k) {
+    const int t = t0 + k;
+    const bool act = lane_on && t < Ttok;
+    const Raw8<T> xr = next[0];
+    float x[8];
+    xr.widen(x);
     if (TAPS > 0) {
+      next[0] = next[1];
+      fetch(k + 2, next[1]);
+    }
+    if (TAPS == 0) {
+      pos = act ? a.tok_pos[t] : 0;
+    } else if (act) {
+      if (k == 0 || t == end) {
+        s = e.tok_seq[t];
+        j = t - e.cu[s];
+        end = e.cu[s + 1];
+        pos = a.tok_pos[t];
+      } else {
+        ++j;
+        ++pos;
+      }
+      if (TAPS > 1) {
+        const T* p = proj + (int64_t)t * a.ld_proj + ch;
+        T* sl = e.tails + (int64_t)e.seq_slot[s] * e.tail_stride + ch;
+        const int C = nq + nk + nv;
+        if (k == 0 || j == 0) {  // (re)load the earlier inputs
+#pragma unroll
+          for (int m = 1; m < TAPS; ++m) {
+            hist[m - 1].zero();
+            if (pos - m >= 0) {
+              if (m <= j)
+                hist[m - 1].load(p - (int64_t)m * a.ld_proj);
+              else
+                hist[m - 1].load(sl + (int64_t)(TAPS - 1 + j - m) * C);
+            }
+          }
+        }
+        if (e.shift_tail) {  // oldest first: x(t-TAPS+2) .. x(t)
+#pragma unroll
+          for (int m = TAPS - 2; m >= 1; --m) hist[m - 1].store(sl + (int64_t)(TAPS - 2 - m) * C);
+          xr.store(sl + (int64_t)(TAPS - 2) * C);
+        }
+      }
+      float w[TAPS > 0 ? 8 * TAPS : 1];  // channel-major: w[channel * TAPS + tap]
 #pragma unroll
       for (int i = 0; i < TAPS; ++i) {
         float tmp[8];
-        load8(e.conv_w + (int64_t)ch * TAPS + 8 * i, tmp);
+        wc[i].keep_packed();
+        wc[i].widen(tmp);
 #pragma unroll
-        for (int u = 0; u < 8; ++u) wc[8 * i + u] = tmp[u];
+        for (int u = 0; u < 8; ++u) w[8 * i + u] = tmp[u];
+      }
+#pragma unroll
+      for (int i = 0; i < 8; ++i) x[i] *= w[i * TAPS + TAPS - 1];
+#pragma unroll
+      for (int m = 1; m < TAPS; ++m) {
+        float hv[8];
+        hist[m - 1].widen(hv);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) x[i] += w[i * TAPS + TAPS - 1 - m] * hv[i];
+      }
+#pragma unroll
+      for (int m = TAPS - 1; m > 1; --m) hist[m - 1] = hist[m - 2];
+      hist[0] = xr;
+    }
+    T* row = a.own_kv && act ? pool + (int64_t)a.tok_row[t] * (nk + nv) : nullptr;
+    if (a.v_from_k && act && !is_q) store8(row + nk + (job - H) * dim + c0, x);
+    // norm in front of the rotation (or of a value head)
+    if (a.norm == 2 || a.v_eps >= 0.f) {
+      float ss = 0.f;
+#pragma unroll
+      for (int i = 0; i < 8; ++i) ss += x[i] * x[i];
+#pragma unroll
+      for (int o = 1; o < LG; o <<= 1) ss += __shfl_xor(ss, o, 64);
+      if (is_v) {
+        if (a.v_eps >= 0.f) {
+          const float inv = rsqrtf(ss / (float)vdim + a.v_eps);
+#pragma unroll
+          for (int i = 0; i < 8; ++i) x[i] *= inv;
+        }
+      } else if (a.norm == 2 && lane_on) {
+        const float inv = rsqrtf(ss / (float)dim + a.eps);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) x[i] *= inv * wv[i];
       }
     }
-    for (int t = t0; t < t1; ++t) {
-      const int pos = a.tok_pos[t];
-      const T* p = proj + (int64_t)t * a.ld_proj;
-      float x[8];
+    if (rot_dims > 0) {
+      const float* cs = a.cosT + (int64_t)pos * half;
+      const float* sn = a.sinT + (int64_t)pos * half;
+      if (a.half) {  // the partner group sits half the rotated width away
+        const int src = (int)(threadIdx.x & 63) - l + (pc >> 3);
+        float o[8];
 #pragma unroll
-      for (int i = 0; i < 8; ++i) x[i] = 0.f;
-      if (act) load8(p + ch, x);
-      if (TAPS > 0) {
-        const int s = e.tok_seq[t], j = t - e.cu[s];
-        if (TAPS > 1) {
-          T* sl = e.tails + (int64_t)e.seq_slot[s] * e.tail_stride + ch;
-          const int C = nq + nk + nv;
-          if (t == t0 || j == 0) {  // block-uniform: (re)load the earlier inputs
+        for (int i = 0; i < 8; ++i) o[i] = __shfl(x[i], src, 64);
+        if (turn) {
+          const int f0 = second ? c0 - half : c0;
+          float co[8], si[8];
+          load8(cs + f0, co);
+          load8(sn + f0, si);
 #pragma unroll
-            for (int k = 1; k < TAPS; ++k) {
-#pragma unroll
-              for (int i = 0; i < 8; ++i) hist[k - 1][i] = 0.f;
-              if (pos - k >= 0 && act) {
-                if (k <= j)
-                  load8(p - (int64_t)k * a.ld_proj + ch, hist[k - 1]);
-                else
-                  load8(sl + (int64_t)(TAPS - 1 + j - k) * C, hist[k - 1]);
-              }
-            }
-          }
-          if (e.shift_tail && act) {  // oldest first: x(t-TAPS+2) .. x(t)
-#pragma unroll
-            for (int k = TAPS - 2; k >= 1; --k)
-              store8(sl + (int64_t)(TAPS - 2 - k) * C, hist[k - 1]);
-            store8(sl + (int64_t)(TAPS - 2) * C, x);
-          }
+          for (int i = 0; i < 8; ++i)
+            x[i] = second ? x[i] * co[i] + o[i] * si[i] : x[i] * co[i] - o[i] * si[i];
         }
-        float y[8];
+      } else if (turn) {
 #pragma unroll
-        for (int i = 0; i < 8; ++i) y[i] = wc[i * TAPS + TAPS - 1] * x[i];
-#pragma unroll
-        for (int k = 1; k < TAPS; ++k)
-#pragma unroll
-          for (int i = 0; i < 8; ++i) y[i] += wc[i * TAPS + TAPS - 1 - k] * hist[k - 1][i];
-#pragma unroll
-        for (int k = TAPS - 1; k >= 1; --k)
-#pragma unroll
-          for (int i = 0; i < 8; ++i) hist[k - 1][i] = k > 1 ? hist[k >= 2 ? k - 2 : 0][i] : x[i];
-#pragma unroll
-        for (int i = 0; i < 8; ++i) x[i] = act ? y[i] : 0.f;
-      }
-      T* row = a.own_kv ? pool + (int64_t)a.tok_row[t] * (nk + nv) : nullptr;
-      if (a.v_from_k && act && !is_q) store8(row + nk + (job - H) * dim + c0, x);
-      // norm in front of the rotation (or of a value head)
-      if (a.norm == 2 || a.v_eps >= 0.f) {
-        float ss = 0.f;
-#pragma unroll
-        for (int i = 0; i < 8; ++i) ss += x[i] * x[i];
-#pragma unroll
-        for (int o = 1; o < LG; o <<= 1) ss += __shfl_xor(ss, o, 64);
-        if (is_v) {
-          if (a.v_eps >= 0.f) {
-            const float inv = rsqrtf(ss / (float)vdim + a.v_eps);
-#pragma unroll
-            for (int i = 0; i < 8; ++i) x[i] *= inv;
-          }
-        } else if (a.norm == 2 && act) {
-          const float inv = rsqrtf(ss / (float)dim + a.eps);
-#pragma unroll
-          for (int i = 0; i < 8; ++i) x[i] *= inv * wv[i];
-        }
-      }
-      if (rot_dims > 0) {
-        const float* cs = a.cosT + (int64_t)pos * half;
-        const float* sn = a.sinT + (int64_t)pos * half;
-        if (a.half) {  // the partner group sits half the rotated width away
-          const int src = (int)(threadIdx.x & 63) - l + (pc >> 3);
-          float o[8];
-#pragma unroll
-          for (int i = 0; i < 8; ++i) o[i] = __shfl(x[i], src, 64);
-          if (turn) {
-            const int f0 = second ? c0 - half : c0;
-            float co[8], si[8];
-            load8(cs + f0, co);
-            load8(sn + f0, si);
-#pragma unroll
-            for (int i = 0; i < 8; ++i)
-              x[i] = second ? x[i] * co[i] + o[i] * si[i] : x[i] * co[i] - o[i] * si[i];
-          }
-        } else if (turn) {
-#pragma unroll
-          for (int i = 0; i < 8; i += 2) {
-            if (c0 + i < rot_dims) {
-              const float co = cs[(c0 + i) >> 1], si = sn[(c0 + i) >> 1];
-              const float u = x[i], v = x[i + 1];
-              x[i] = u * co - v * si;
-              x[i + 1] = v * co + u * si;
-            }
+        for (int i = 0; i < 8; i += 2) {
+          if (c0 + i < rot_dims) {
+            const float co = cs[(c0 + i) >> 1], si = sn[(c0 + i) >> 1];
+            const float u = x[i], v = x[i + 1];
+            x[i] = u * co - v * si;
+            x[i + 1] = v * co + u * si;
           }
         }
       }
-      float f = is_q && a.qfac ? a.qfac[pos] : 1.f;
-      if (a.norm == 3) {
-        float ss = 0.f;
+    }
+    float f = is_q && a.qfac ? a.qfac[pos] : 1.f;
+    if (a.norm == 3) {
+      float ss = 0.f;
 #pragma unroll
-        for (int i = 0; i < 8; ++i) ss += x[i] * x[i];
+      for (int i = 0; i < 8; ++i) ss += x[i] * x[i];
 #pragma unroll
-        for (int o = 1; o < LG; o <<= 1) ss += __shfl_xor(ss, o, 64);
-        if (!is_v) f *= rsqrtf(ss / (float)dim + a.eps);
-      }
-      if (!act) continue;
+      for (int o = 1; o < LG; o <<= 1) ss += __shfl_xor(ss, o, 64);
+      if (!is_v) f *= rsqrtf(ss / (float)dim + a.eps);
+    }
+    if (act) {
 #pragma unroll
       for (int i = 0; i < 8; ++i) x[i] *= f;
       store8(is_q ? q_out + (int64_t)t * nq + job * dim + c0
@@ -2006,7 +2074,7 @@ int dsv_window_attn(const void* q, const void* pool, const int* tok_seq, const i
                     float scale, int window, int keep_first, int chunk, float softcap,
                     float out_scale, const float* sink, const void* gate, int ld_gate,
                     hipStream_t s) {
-  if (vdim > WVPT * NT || H % G || nsplit < 1 || (nsplit > 1 && !part)) return -1;
+  if (vdim > WVPT * NT || H % G || nsplit < 1 || nsplit > 64 || (nsplit > 1 && !part)) return -1;
   if ((window > 0 && chunk > 0) || ld_out < H * vdim || (gate && ld_gate < H)) return -3;
   if (Ttok <= 0) return 0;
   const int64_t lds = dsv_window_attn_lds(dt, dim, vdim, KC);
@@ -2018,7 +2086,7 @@ int dsv_window_attn(const void* q, const void* pool, const int* tok_seq, const i
                    nsplit > 1 ? 1.f : out_scale, sink, (const T*)gate, ld_gate)));
   if (nsplit > 1) {
     dim3 g2(Ttok, H);
-    BY_DTYPE(dt, (window_attn_merge_k<T><<<g2, NT, 0, s>>>(
+    BY_DTYPE(dt, (window_attn_merge_k<T><<<g2, merge_threads(vdim), 0, s>>>(
                      part, (T*)out, ld_out, H, vdim, nsplit, out_scale, sink, (const T*)gate,
                      ld_gate)));
   }
@@ -2042,7 +2110,7 @@ int dsv_window_attn_mfma(const void* q, const void* pool, const int* work, int n
                          const void* gate, int ld_gate, hipStream_t s) {
   if (!dsv_window_attn_mfma_ok(dim, vdim) || H % G) return -1;
   if ((window > 0 && chunk > 0) || ld_out < H * vdim || (gate && ld_gate < H)) return -4;
-  if (nsplit < 1 || (nsplit > 1 && !part)) return -3;
+  if (nsplit < 1 || nsplit > 64 || (nsplit > 1 && !part)) return -3;
   if (nwork <= 0) return 0;
 #define GO(DKT, DVB, PF)                                                                        \
   return launch_window_attn_mfma<DKT, DVB, PF>(q, pool, work, nwork, cu, seq_start, table, maxb, \
@@ -2087,7 +2155,7 @@ int dsv_delta_prep(const void* proj, int ld_proj, const void* w, void* state,
                    seq_slot, tok_seq, tok_pos, a_log, dt_bias, q_out, k_out, v_out, beta, decay,
                    G, H, dim, vdim, taps, beta_col, a_col)));
   if (taps > 1)
-    BY_DTYPE(dt, (conv_tail_shift_k<T><<<nseq, NT, 0, s>>>((const T*)proj, ld_proj, (T*)state,
+    BY_DTYPE(dt, (conv_tail_shift_k<T><<<dim3(nseq, (C + NT - 1) / NT), NT, 0, s>>>((const T*)proj, ld_proj, (T*)state,
                                                            state_slot_stride, cu, seq_slot,
                                                            seq_start, C, taps)));
   return (int)hipGetLastError();
@@ -2218,10 +2286,10 @@ int dsv_softplus_decay(const void* z, int ld_z, const float* bias, const float* 
   return (int)hipGetLastError();
 }
 
-// 1 when the vector form of the per-head prologue covers these operands: whole
+// whether the vector form of the per-head prologue covers these operands: whole
 // groups of 8 everywhere; with the half pairing a group's partner is a whole
 // group too. The convolution and the side activation exist in it only.
-int dsv_attn_prep_heads_vec(int ld_proj, int dim, int vdim, int rot_dims, int half, int taps) {
+static int attn_prep_heads_vec(int ld_proj, int dim, int vdim, int rot_dims, int half, int taps) {
   const int big = dim > vdim ? dim : vdim;
   return dim % 8 == 0 && vdim % 8 == 0 && ld_proj % 8 == 0 && big <= 512 &&
          (half ? rot_dims % 16 == 0 : 1) && taps >= 0 && taps <= 4 && taps != 1;
@@ -2248,7 +2316,7 @@ int dsv_attn_prep_heads(const void* proj, int ld_proj, const float* wq, const fl
   if (v_from_k && (!own_kv || dim != vdim || taps > 0 || v_eps >= 0.f)) return -4;
   const int C = H * dim + (own_kv ? G * dim + (v_from_k ? 0 : G * vdim) : 0);
   if (ld_proj < C) return -5;
-  const bool vec = dsv_attn_prep_heads_vec(ld_proj, dim, vdim, rot_dims, half, taps) &&
+  const bool vec = attn_prep_heads_vec(ld_proj, dim, vdim, rot_dims, half, taps) &&
                    (uintptr_t)proj % 16 == 0;
   const bool extra = taps > 0 || side_n > 0;
   if (extra && !vec) return -6;
@@ -2266,17 +2334,17 @@ int dsv_attn_prep_heads(const void* proj, int ld_proj, const float* wq, const fl
   }
   const int big = dim > vdim ? dim : vdim;
   const int jobs = own_kv ? (v_from_k ? H + G : H + 2 * G) : H;
-  const bool few = Ttok < 512;  // spread a token's heads over workgroups
-  const int toks = taps > 0 && !few ? 4 : 1;
-  const int blocks = (Ttok + toks - 1) / toks;
+  const int toks = taps > 0 && Ttok >= 512 ? PREP_TOKS : 1;
+  const int64_t units = (int64_t)((Ttok + toks - 1) / toks) * jobs;
+  const int64_t side8 = side_n > 0 ? (int64_t)Ttok * (side_n / 8) : 0;
+  if (units > (1 << 26) || side8 > (int64_t)1 << 30) return -9;
 #define PREPV(LG, TAPS)                                                                           \
   do {                                                                                            \
-    const int ny = few ? (jobs + NT / LG - 1) / (NT / LG) : 1;                                    \
-    const int ns = side_n > 0 ? (few ? (side_n / 8 + NT - 1) / NT : 1) : 0;                       \
-    BY_DTYPE(dt, (attn_prep_heads_vec_k<T, LG, TAPS><<<dim3(blocks, ny + ns), NT, 0, s>>>(        \
+    const int np = (int)((units + NT / LG - 1) / (NT / LG)), ns = (int)((side8 + NT - 1) / NT);   \
+    BY_DTYPE(dt, (attn_prep_heads_vec_k<T, LG, TAPS><<<np + ns, NT, 0, s>>>(                      \
                      (const T*)proj, (T*)pool, (T*)q_out, Ttok, a,                                \
                      PrepSteps<T>{(const T*)conv_w, (T*)tails, tail_stride, cu, seq_slot,         \
-                                  tok_seq, single, toks, ny, (const T*)side_in, (T*)side_out,     \
+                                  tok_seq, single, toks, np, (const T*)side_in, (T*)side_out,     \
                                   side_n, side_ld_in, side_ld_out})));                            \
   } while (0)
 #define PREPV_BY_LG(TAPS)                  \
@@ -2294,7 +2362,7 @@ int dsv_attn_prep_heads(const void* proj, int ld_proj, const float* wq, const fl
 #undef PREPV_BY_LG
 #undef PREPV
   if (taps > 1 && !single)
-    BY_DTYPE(dt, (conv_tail_shift_k<T><<<nseq, NT, 0, s>>>((const T*)proj, ld_proj, (T*)tails,
+    BY_DTYPE(dt, (conv_tail_shift_k<T><<<dim3(nseq, (C + NT - 1) / NT), NT, 0, s>>>((const T*)proj, ld_proj, (T*)tails,
                                                            tail_stride, cu, seq_slot, seq_start,
                                                            C, taps)));
   return (int)hipGetLastError();
@@ -2336,7 +2404,7 @@ int dsv_conv_silu(const void* x, int ld_x, const void* w, const float* bias, voi
                      (const T*)x, ld_x, (const T*)w, bias, (const T*)state, state_slot_stride,
                      cu, seq_slot, tok_seq, tok_pos, (T*)out, C, taps, silu)));
   if (taps > 1)
-    BY_DTYPE(dt, (conv_tail_shift_k<T><<<nseq, NT, 0, s>>>((const T*)x, ld_x, (T*)state,
+    BY_DTYPE(dt, (conv_tail_shift_k<T><<<dim3(nseq, (C + NT - 1) / NT), NT, 0, s>>>((const T*)x, ld_x, (T*)state,
                                                            state_slot_stride, cu, seq_slot,
                                                            seq_start, C, taps)));
   return (int)hipGetLastError();
@@ -2371,7 +2439,7 @@ int dsv_ssd_prep(const void* proj, int ld_proj, const void* w, const float* bias
                    state_slot_stride, cu, seq_slot, tok_seq, tok_pos, a_log, dt_bias, x_out,
                    v_out, b_out, c_out, decay, H, P, G, N, taps)));
   if (taps > 1)
-    BY_DTYPE(dt, (conv_tail_shift_k<T><<<nseq, NT, 0, s>>>(
+    BY_DTYPE(dt, (conv_tail_shift_k<T><<<dim3(nseq, (C + NT - 1) / NT), NT, 0, s>>>(
                      (const T*)proj + inner, ld_proj, (T*)state, state_slot_stride, cu, seq_slot,
                      seq_start, C, taps)));
   return (int)hipGetLastError();

@@ -98,12 +98,35 @@ def load(which="rows"):
         lib = _libs[which] = ctypes.CDLL(build(force=False, which=which))
         if which == "latent":
             lib.dsv_latent_attn_lds.restype = ctypes.c_int64
+        if which == "seq":
+            lib.dsv_window_attn_lds.restype = ctypes.c_int64
+        for name, kinds in _SIGNATURES.get(which, {}).items():
+            getattr(lib, name).argtypes = [_KINDS[k] for k in kinds]
     return lib
 
 
+# Entry points called many times per step declare their arguments (p: pointer
+# or None, i: int, l: int64, f: float), so that plain Python numbers are
+# converted by ctypes itself: decode steps are bound by the host.
+_KINDS = {"p": ctypes.c_void_p, "i": ctypes.c_int, "l": ctypes.c_int64,
+          "f": ctypes.c_float}
+_SIGNATURES = {
+    "rows": {"dsv_residual_tanh": "ppi" + "p" * 5 + "iiip"},
+    "seq": {"dsv_attn_prep_heads": "pi" + "p" * 9 + "i" * 11 + "ff"
+                                   + "ppli" + "pppp" + "ii" + "pipii" + "p",
+            "dsv_window_attn_mfma": "pppi" + "ppp" + "ii" + "pip" + "i" * 6
+                                    + "fiiiff" + "ppi" + "p"},
+}
+
+
+_has_gpu = None
+
+
 def enabled() -> bool:
-    return torch.cuda.is_available() and \
-        os.environ.get("DS_AMD_SERVING_EAGER") != "1"
+    global _has_gpu
+    if _has_gpu is None:
+        _has_gpu = torch.cuda.is_available()
+    return _has_gpu and os.environ.get("DS_AMD_SERVING_EAGER") != "1"
 
 
 _DT = {torch.float32: 0, torch.bfloat16: 1}
@@ -123,8 +146,18 @@ def _p(t):
     return ctypes.c_void_p(t.data_ptr())
 
 
+def _at(t):
+    """Address of a contiguous device tensor (None passes) for an entry point
+    with declared arguments."""
+    if t is None:
+        return None
+    assert t.is_cuda and t.is_contiguous(), "kernel operands are contiguous device tensors"
+    return t.data_ptr()
+
+
 def _stream():
-    return ctypes.c_void_p(torch.cuda.current_stream().cuda_stream)
+    return ctypes.c_void_p(torch._C._cuda_getCurrentRawStream(
+        torch.cuda.current_device()))
 
 
 def _f(x):
@@ -483,9 +516,7 @@ def grouped_topk(logits, correction, top, groups, keep, score, group_score,
 
 # ------------------------------------------------------ windowed attention
 def _seq():
-    lib = load("seq")
-    lib.dsv_window_attn_lds.restype = ctypes.c_int64
-    return lib
+    return load("seq")
 
 
 def _rows_ok(t):
@@ -547,9 +578,10 @@ def attn_prep(proj, batch, pool, q_norm_w, k_norm_w, eps, heads, kv_heads,
     if q_factor is not None:
         assert q_factor.dtype == torch.float32 and q_factor.dim() == 1
         assert q_factor.numel() >= batch.max_ctx
-    vec = proj.data_ptr() % 16 == 0 and lib.dsv_attn_prep_heads_vec(
-        _i(proj.stride(0)), _i(dim), _i(vdim), _i(rot_dims), _i(half),
-        _i(taps)) == 1
+    # the vector form's sizes (dsv_attn_prep_heads refuses what it cannot do)
+    vec = dim % 8 == 0 and vdim % 8 == 0 and max(dim, vdim) <= 512 and \
+        rot_dims % (16 * half or 1) == 0 and taps != 1 and taps <= 4 and \
+        proj.stride(0) % 8 == 0 and proj.data_ptr() % 16 == 0
     if taps and not vec:        # sizes the fused form does not cover
         proj = conv_silu_ragged(proj, conv_w, tails, batch, None, proj.dtype,
                                 None)
@@ -562,26 +594,22 @@ def attn_prep(proj, batch, pool, q_norm_w, k_norm_w, eps, heads, kv_heads,
         else:
             assert z.shape == z_out.shape and z.shape[0] == T
             assert z.dtype == z_out.dtype == proj.dtype
+    head = norm == "head"
     _check(lib.dsv_attn_prep_heads(
-        _vp(proj), _i(proj.stride(0)),
-        _p(_f32(q_norm_w) if norm == "head" else None),
-        _p(_f32(k_norm_w) if norm == "head" and own_kv else None),
-        _p(batch.tok_pos), _p(batch.tok_row), _p(cos if rot_dims else None),
-        _p(sin if rot_dims else None), _p(q_factor), _p(pool), _p(q),
-        _i(_dt(proj)), _i(T), _i(heads), _i(kv_heads), _i(dim), _i(vdim),
-        _i(rot_dims), _i(1 if own_kv else 0),
-        _i({None: 0, "head": 2, "after": 3}[norm]), _i(half),
-        _i(1 if v_from_k else 0), _f(eps),
-        _f(-1.0 if v_unit_eps is None else v_unit_eps),
-        _p(conv_w if taps else None), _vp(tails) if taps else _p(None),
-        _l(tails.stride(0) if taps else 0), _i(taps), _p(batch.cu),
-        _p(batch.seq_slot), _p(batch.seq_start), _p(batch.tok_seq),
-        _i(batch.n_seqs), _i(1 if single_tokens(batch) else 0),
-        _p(None) if side is None else _vp(z),
-        _i(0 if side is None else z.stride(0)),
-        _p(None) if side is None else _vp(z_out),
-        _i(0 if side is None else z_out.stride(0)),
-        _i(0 if side is None else z.shape[1]), _stream()), "attn_prep_heads")
+        proj.data_ptr(), proj.stride(0), _at(_f32(q_norm_w)) if head else None,
+        _at(_f32(k_norm_w)) if head and own_kv else None, _at(batch.tok_pos),
+        _at(batch.tok_row), _at(cos) if rot_dims else None,
+        _at(sin) if rot_dims else None, _at(q_factor), _at(pool), _at(q),
+        _dt(proj), T, heads, kv_heads, dim, vdim, rot_dims,
+        1 if own_kv else 0, {None: 0, "head": 2, "after": 3}[norm], half,
+        1 if v_from_k else 0, eps, -1.0 if v_unit_eps is None else v_unit_eps,
+        _at(conv_w) if taps else None, tails.data_ptr() if taps else None,
+        tails.stride(0) if taps else 0, taps, _at(batch.cu),
+        _at(batch.seq_slot), _at(batch.seq_start), _at(batch.tok_seq),
+        batch.n_seqs, 1 if single_tokens(batch) else 0,
+        *((None, 0, None, 0, 0) if side is None else
+          (z.data_ptr(), z.stride(0), z_out.data_ptr(), z_out.stride(0),
+           z.shape[1])), _stream()), "attn_prep_heads")
     return q
 
 
@@ -645,8 +673,8 @@ def window_attention(q, pool, batch, kv_heads, dim, vdim, scale, window=0,
     if gate is not None:
         assert gate.shape == (T, H) and gate.dtype == q.dtype
         _rows_ok(gate)
-    extra = (_p(sink), _p(None) if gate is None else _vp(gate),
-             _i(0 if gate is None else gate.stride(0)))
+    extra = (_at(sink), None if gate is None else gate.data_ptr(),
+             0 if gate is None else gate.stride(0))
     mfma = q.dtype == torch.bfloat16 and \
         lib.dsv_window_attn_mfma_ok(_i(dim), _i(vdim)) == 1
     if path is None:
@@ -666,12 +694,11 @@ def window_attention(q, pool, batch, kv_heads, dim, vdim, scale, window=0,
             part = torch.empty(T, nsplit, H, vdim + 2, dtype=torch.float32,
                                device=q.device)
         _check(lib.dsv_window_attn_mfma(
-            _p(q), _p(pool), _p(work), _i(n), _p(batch.cu),
-            _p(batch.seq_start), _p(batch.block_table),
-            _i(batch.block_table.shape[1]), _i(batch.block_size), _vp(out),
-            _i(ld_out), _p(part), _i(T), _i(H), _i(kv_heads), _i(dim),
-            _i(vdim), _i(nsplit), _f(scale), _i(window), _i(keep_first),
-            _i(chunk), _f(softcap), _f(out_scale), *extra, _stream()),
+            _at(q), _at(pool), _at(work), n, _at(batch.cu),
+            _at(batch.seq_start), _at(batch.block_table),
+            batch.block_table.shape[1], batch.block_size, out.data_ptr(),
+            ld_out, _at(part), T, H, kv_heads, dim, vdim, nsplit, scale,
+            window, keep_first, chunk, softcap, out_scale, *extra, _stream()),
             "window_attention(mfma)")
         return out
     kc = 64
@@ -693,7 +720,8 @@ def window_attention(q, pool, batch, kv_heads, dim, vdim, scale, window=0,
         _i(batch.block_size), _vp(out), _i(ld_out), _p(part), _i(dt), _i(T),
         _i(H), _i(kv_heads), _i(dim), _i(vdim), _i(kc), _i(nsplit), _f(scale),
         _i(window), _i(keep_first), _i(chunk), _f(softcap), _f(out_scale),
-        *extra, _stream()), "window_attention")
+        _p(sink), ctypes.c_void_p(extra[1]), _i(extra[2]), _stream()),
+        "window_attention")
     return out
 
 
@@ -1096,9 +1124,9 @@ def residual_tanh(x, y, alpha, weight, bias, out_dtype, index):
         rows = index.numel()
     h = torch.empty(rows, C, dtype=out_dtype, device=x.device)
     _check(load().dsv_residual_tanh(
-        _p(x), _p(y), _i(0 if y is None else _dt(y)), _p(_f32(alpha)),
-        _p(_f32(weight).contiguous()), _p(_f32(bias).contiguous()), _p(index),
-        _p(h), _i(_DT[out_dtype]), _i(rows), _i(C), _stream()),
+        _at(x), _at(y), 0 if y is None else _dt(y), _at(_f32(alpha)),
+        _at(_f32(weight).contiguous()), _at(_f32(bias).contiguous()),
+        _at(index), _at(h), _DT[out_dtype], rows, C, _stream()),
         "residual_tanh")
     return h
 

@@ -906,6 +906,24 @@ def test_http_server_generates_the_oracles_tokens():
         assert g == seq[len(p):]
 
 
+def test_declared_kernel_arguments_match_the_sources():
+    """Entry points whose argument kinds Python declares: as the C source
+    has them."""
+    import re
+    from deepspeed_amd.ops import serving_kernels as sk
+    for lib, table in sk._SIGNATURES.items():
+        with open(sk.LIBRARIES[lib][0]) as f:
+            src = f.read()
+        for name, kinds in table.items():
+            args = re.search(r"int %s\((.*?)\)\s*\{" % name, src, re.S)
+            got = ""
+            for a in args.group(1).split(","):
+                a = a.strip()
+                got += "p" if "*" in a or "hipStream_t" in a else \
+                    "l" if "int64_t" in a else "f" if "float" in a else "i"
+            assert got == kinds, name
+
+
 # ------------------------------------------- HIP kernels against eager ops
 @pytest.mark.gpu
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])

@@ -993,7 +993,7 @@ def near(got, want, dtype):
 
 @pytest.mark.gpu
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
-@pytest.mark.parametrize("C", [1, 13, 24, 192, 520, 1000, 4096, 4099, 8192])
+@pytest.mark.parametrize("C", [1, 13, 24, 200, 520, 1000, 4096, 4099, 8192])
 def test_dynamic_tanh_kernel_against_eager(C, dtype, monkeypatch):
     from deepspeed_amd.ops.norms import residual_tanh
     al = torch.tensor([0.4]).to(DEV)
@@ -1028,11 +1028,11 @@ def test_relu_squared_kernel_against_eager(dtype, monkeypatch):
 
 
 PREPS = [  # heads, kv, dim, vdim, rotated, layout, norm, taps, keys as values
-    (4, 2, 64, 64, 16, "interleaved", "after", 0, True),
+    (6, 2, 64, 64, 32, "interleaved", "after", 0, True),
     (4, 2, 10, 10, 8, "interleaved", "after", 0, True),
     (8, 1, 128, 128, 128, "half", "after", 0, True),
     (3, 3, 24, 24, 6, "interleaved", "after", 0, True),
-    (4, 1, 96, 96, 48, "half", None, 3, False),
+    (6, 2, 80, 88, 48, "half", None, 3, False),
     (4, 2, 96, 40, 32, "half", None, 4, False),
     (2, 2, 16, 24, 16, "half", None, 2, False),
     (2, 1, 256, 128, 64, "half", "head", 4, False),
@@ -1097,7 +1097,7 @@ def test_prologue_kernel_against_eager(H, G, d, dv, dims, layout, norm, taps,
 @pytest.mark.gpu
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 @pytest.mark.parametrize("H,G,d,dv,window,keep", [
-    (4, 2, 64, 64, 70, 3), (4, 1, 96, 96, 0, 0), (8, 2, 128, 128, 0, 0),
+    (6, 2, 64, 64, 70, 3), (4, 1, 80, 96, 0, 0), (8, 2, 128, 128, 0, 0),
     (3, 3, 20, 12, 9, 2), (6, 1, 200, 130, 0, 0), (2, 1, 16, 24, 300, 40)])
 def test_attention_kernels_with_sink_and_gate(H, G, d, dv, window, keep,
                                               dtype, monkeypatch):
